@@ -42,7 +42,7 @@ int nvs_norm_residual(const void* m, const void* m2, const void* w1, const void*
 
 /* Input-side norm on the residual stream, with the adds that precede it: x[t, :] += a_mult * a[t, :] + b[t, :] (a in `dtype`,
  * b 32-bit, either may be NULL), then out[t, :] = group_rms(x[t, :]) * w: every one of `groups` equal consecutive parts of the
- * row is divided by its own sqrt(mean(part^2) + eps); with center != 0 the part's mean is taken off first and it is divided by
+ * row is divided by its own sqrt(mean(part^2) + eps) (w == NULL: out is the sum itself, rounded to `dtype`); with center != 0 the part's mean is taken off first and it is divided by
  * sqrt(mean of squared deviations + eps) (a layer norm without bias). out == NULL: the adds only. With rows != NULL nothing is
  * added and out[r, :] is the norm of x[rows[r], :]. out and w in `dtype`. */
 int nvs_add_group_norm(float* x, const void* a, float a_mult, const float* b, const int32_t* rows, int64_t nrows, const void* w,
@@ -55,6 +55,21 @@ int nvs_add_group_norm(float* x, const void* a, float a_mult, const float* b, co
  * norm of x[rows[r], :]. a, a2, wa, w, out in `dtype`; every sum in 32-bit. */
 int nvs_sandwich_norm(float* x, const void* a, float a_mult, const void* a2, float a2_mult, const void* wa, const int32_t* rows,
                       int64_t nrows, const void* w, float w_off, int dtype, int width, float eps, void* out, void* stream);
+
+/* x[t, :] = rms(table[ids[t], :]) * w, 32-bit. */
+int nvs_embed_norm(const void* table, int dtype, const int64_t* ids, int64_t n, int width, const void* w, float eps, float* x, void* stream);
+
+/* Input-side norm with a token shift, and the add before it. y[t, :] = x[t, :] + a[t, :] (wa NULL) or x[t, :] + rms(a[t, :]) * wa, written to
+ * x_out (a NULL: y = x and x_out may be x); h[t, :] = rms(y[t, :]) * w; out[t, :] = h[t, :] + (h[t - 1, :] - h[t, :]) * mu, where the row
+ * before a portion's first one is the state [nslots, width] (32-bit; zeros at a sequence's start), which the portion's last h replaces.
+ * x_out must not be x when a is given. All in 32-bit; a, wa, w, mu, out in `dtype`. */
+int nvs_shift_norm(const float* x, const void* a, const void* wa, const void* w, const void* mu, int dtype, const int32_t* cu_q,
+                   const int32_t* ctx0, const int32_t* slot, const int32_t* tseq, int nseq, int64_t n, int width, float eps, float* state,
+                   float* x_out, void* out, void* stream);
+
+/* A gated lookup: out[t, c] = gelu_tanh(z[t, c]) * table[ids[t], col0 + c], c < dim (z row stride z_stride, table row stride table_stride). */
+int nvs_gated_lookup(const void* z, int64_t z_stride, const void* table, int64_t table_stride, int64_t col0, int dtype, const int64_t* ids, int dim,
+                     int64_t n, void* out, void* stream);
 
 /* out[i] = cap * tanh(in[i] * scale / cap), or in[i] * scale with cap <= 0; in `dtype`, out 32-bit. */
 int nvs_scale_softcap(const void* in, int dtype, float scale, float cap, int64_t numel, float* out, void* stream);
@@ -127,11 +142,27 @@ int nvs_gated_memory_scan(const void* proj, int64_t proj_stride, int64_t v_col, 
                           float* M, float* y, float* den, float* ws, int64_t ws_floats, void* stream);
 
 /* order 0: out = group_rms(y * silu(z)) * w: the gate first, then each of `groups` equal parts of a row by its own root mean
- * square. order 1: out = group_rms(y) * w * sigmoid(z): the norm first. y [n, inner] 32-bit; z [n, inner] with row stride z_stride
- * (`dtype`); w [inner]; out [n, inner] `dtype`. den (nullable, order 1 only) [n, groups] 32-bit: every entry of group g of row t is
+ * square. order 1: out = group_rms(y) * w * sigmoid(z): the norm first; order 2: out = group_rms(y) * w * silu(z). y [n, inner] 32-bit;
+ * z [n, inner] with row stride z_stride (`dtype`); w [wlen], wlen = inner or, shared by the groups, inner / groups; out [n, inner]
+ * `dtype`. den (nullable, order 1 and 2) [n, groups] 32-bit: every entry of group g of row t is
  * divided by den[t, g] first. */
-int nvs_gated_group_norm(const float* y, const void* z, int64_t z_stride, int dtype, const void* w, int inner, int groups,
+int nvs_gated_group_norm(const float* y, const void* z, int64_t z_stride, int dtype, const void* w, int wlen, int inner, int groups,
                          float eps, int order, int64_t n, const float* den, void* out, void* stream);
+
+/* The gated delta rule, in 32-bit. Per head h, token by token, with unit vectors q, k (per group of heads), a value v, a step size
+ * beta and decays g:   S <- g * S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q.
+ * qkv [n, qkv_stride] (`dtype`): q | k (G x dk each) | v (heads x dv), after convolution and activation; head h uses group
+ * h / (heads / G). Here q and k become x / sqrt(sum(x^2) + 1e-6), q also times q_scale. beta = sigmoid(column b_col + h of gates
+ * [n, gates_stride] (`dtype`)). per_channel == 0: one decay per head, g = exp(-exp(A_log[h]) softplus(column a_col + h of gates +
+ * dt_bias[h])); per_channel != 0: one per head and key channel from columns a_col + h dk + c of `decays` [n, decays_stride] and dt_bias
+ * [heads * dk]. A_log and dt_bias 32-bit. State S [nslots, heads, dv, dk] (dk fastest), advanced. y [n, heads * dv] 32-bit.
+ * Long portions are walked in chunks of 16 tokens on the 32-bit matrix cores (a triangular system per chunk); steps of short portions
+ * token by token. nvs_delta_force: tests / A-B, 1 always token by token, 2 always in chunks, 0 the default. */
+int nvs_delta_scan(const void* qkv, int64_t qkv_stride, const void* gates, int64_t gates_stride, int64_t b_col, int64_t a_col,
+                   const void* decays, int64_t decays_stride, int dtype, const float* A_log, const float* dt_bias, float q_scale,
+                   int per_channel, int heads, int G, int dk, int dv, const int32_t* cu_q, const int32_t* ctx0, const int32_t* slot, int nseq,
+                   int64_t n, int64_t max_q, float* S, float* y, void* stream);
+void nvs_delta_force(int mode);
 
 /* Key norm / rotation + paged K/V store. Rotation (rot_dims > 0, after the norm): entries (2i, 2i+1), i < rot_dims / 2, of every key head turn by
  * the angle pos[t] * rot_freq[i] (32-bit): (u, v) -> (u cos - v sin, v cos + u sin); the other entries pass. k [n, G, d] / v [n, G, dv] are column ranges of one projection output (row stride `stride`,
@@ -151,14 +182,35 @@ int nvs_knorm_kvstore(const void* k, const void* v, int64_t stride, int dtype, c
  * * (1 + qt_coef * ln(floor((p + 1) / qt_every) + 1)) (qt_every == 0: no such factor), softmax in 32-bit; with sink != NULL ([H],
  * 32-bit) the denominator of head h also holds exp(sink[h]), a score that is not scaled and has no value. gate (nullable) [n, H*dv] with row stride
  * gate_stride: out *= sigmoid(gate); with gate_per_head != 0 the gate is [n, H], one entry for all columns of a head. out [n, H*dv] `dtype`.
+ * q_row (nullable, [n] 32-bit): query row t is multiplied by q_row[t] and by qnorm [H * d] instead (a norm over the whole projection).
+ * softcap > 0: score <- softcap * tanh(score / softcap). pool > 0 (behind a window): beside the window's tokens a query sees one key
+ * and value for every block of `pool` positions that lies wholly before its window (nvs_pool_blocks), in the same softmax.
  * bf16 with d % 8 == 0, d and dv <= 256 and block_size % 8 == 0 runs on the matrix cores (16 queries per wavefront — 16 positions of
  * one head, or in steps of single tokens with 8 or more query heads per kv head 16 heads at one position; the weights enter the
  * second product as bf16); everything else, and every float32 call, takes the scalar kernel (one wavefront per query). */
-int nvs_window_attn(const void* q, int64_t q_stride, const void* qnorm, float eps, const void* gate, int64_t gate_stride, int gate_per_head, int dtype,
-                    const void* k_cache, const void* v_cache, const int32_t* block_tables, int64_t bt_stride, int block_size,
-                    const int32_t* cu_q, const int32_t* ctx0, const int32_t* tseq, int nseq, int64_t n, int H, int G, int d, int dv,
-                    float scale, int window, int chunk, const float* rot_freq, int rot_dims, const float* sink, float qt_coef, int qt_every,
-                    void* out, void* stream);
+int nvs_window_attn(const void* q, int64_t q_stride, const void* qnorm, float eps, const float* q_row, const void* gate,
+                    int64_t gate_stride, int gate_per_head, int dtype, const void* k_cache, const void* v_cache,
+                    const int32_t* block_tables, int64_t bt_stride, int block_size, const int32_t* cu_q, const int32_t* ctx0,
+                    const int32_t* tseq, int nseq, int64_t n, int H, int G, int d, int dv, float scale, float softcap, int window,
+                    int chunk, int pool, const void* pool_k, const void* pool_v, const float* rot_freq, int rot_dims,
+                    const float* sink, float qt_coef, int qt_every, void* out, void* stream);
+
+/* Norm over WHOLE query / key projections, with the paged store. q [n, q_cols] (row stride q_stride): q_row[t] = 1 / sqrt(mean(q[t]^2)
+ * + eps), the factor that nvs_window_attn multiplies in. k (nullable) [n, G * d], v [n, G * dv] (row stride `stride`): the key row is
+ * divided by its root mean square, multiplied by knorm [G * d], rotated per head and stored with v as nvs_knorm_kvstore does. With
+ * pool > 0 and finish != 0 (every portion of the step is ONE token) the means of the blocks that the step completes are taken too. */
+int nvs_qk_rows(const void* q, int64_t q_stride, int q_cols, const void* k, const void* v, int64_t stride, int dtype, const void* knorm,
+                float eps, int G, int d, int dv, int block_size, const int32_t* slots, const int64_t* pos, const float* rot_freq, int rot_dims,
+                int64_t n, float* q_row, void* k_cache, void* v_cache, int pool, int finish, const int32_t* block_tables, int64_t bt_stride,
+                const int32_t* tseq, void* pool_k, void* pool_v, void* stream);
+
+/* Means over blocks of `pool` tokens, b P .. b P + P - 1, of the cached keys and values: every block whose last token is a row of this
+ * step (rows with slots[t] < 0 are skipped). pool_k [pages * nvs_pool_rows][G][d], pool_v [pages * nvs_pool_rows / 8][G][dv][8]: blocks
+ * are kept in units of 8, unit u in the page that holds position 8 u P + P - 1; nvs_pool_rows(block_size, pool) blocks per page. */
+int64_t nvs_pool_rows(int block_size, int pool);
+int nvs_pool_blocks(const void* k_cache, const void* v_cache, int dtype, int G, int d, int dv, int block_size, int pool, const int32_t* slots,
+                    const int64_t* pos, const int32_t* block_tables, int64_t bt_stride, const int32_t* tseq, int64_t n, void* pool_k,
+                    void* pool_v, void* stream);
 
 /* Gated feed-forward activation on a fused [gate | up] projection: gu [n, 2 ff] with row stride `stride` -> out [n, ff] (`dtype`).
  * kind 0: silu(g) u. kind 1: g' = min(g, limit), u' = clamp(u, -limit, limit), out = g' sigmoid(alpha g') (u' + 1).
@@ -193,11 +245,12 @@ int nvs_moe_gemm(const void* X, int64_t ldx, const void* W, int dtype, int mode,
 /* tests: 1 routes bf16 calls through the plain kernel as well */
 void nvs_moe_force_plain(int on);
 
-/* out[t, :] = sum_k wts[t, k] * (pair_row[t, k] >= 0 ? rows[pair_row[t, k], :] : h[t, :]) + sigmoid(shared_gate[t]) * shared[t, :]
+/* With res != NULL ([n, width] 32-bit) the sum is added to it, res += ..., and out (nullable then) receives the new res in `dtype`.
+ * out[t, :] = sum_k wts[t, k] * (pair_row[t, k] >= 0 ? rows[pair_row[t, k], :] : h[t, :]) + sigmoid(shared_gate[t]) * shared[t, :]
  * (shared NULL: no shared expert; shared_gate 32-bit pre-activations with row stride gate_stride, NULL: the shared expert is added
  * as it is). */
 int nvs_moe_combine(const void* rows, int64_t ldr, const int32_t* pair_row, const float* wts, int top, const void* h, int64_t ldh,
-                    const void* shared, const float* shared_gate, int64_t gate_stride, int dtype, int64_t n, int width, void* out,
+                    const void* shared, const float* shared_gate, int64_t gate_stride, int dtype, int64_t n, int width, float* res, void* out,
                     void* stream);
 
 /* Latent attention, around the attention call (nvs_window_attn with one kv head of size kv_rank + rot_dim, values = the latent).

@@ -412,7 +412,7 @@ template <typename T>
 __global__ void moe_combine_kernel(const T* __restrict__ rows, int64_t ldr, const int32_t* __restrict__ pair_row,
                                    const float* __restrict__ wts, int top, const T* __restrict__ h, int64_t ldh,
                                    const T* __restrict__ shared, const float* __restrict__ shared_gate, int64_t gate_stride, int width,
-                                   T* __restrict__ out) {
+                                   float* __restrict__ res, T* __restrict__ out) {
   const int64_t t = blockIdx.x;
   float sg = 0.f;
   if (shared) sg = shared_gate ? 1.f / (1.f + expf(-shared_gate[t * gate_stride])) : 1.f;      // no gate: the shared expert is added as it is
@@ -424,7 +424,11 @@ __global__ void moe_combine_kernel(const T* __restrict__ rows, int64_t ldr, cons
       acc += wts[t * top + k] * v;
     }
     if (shared) acc += sg * ldf(shared + t * width + c);
-    stf(out + t * width + c, acc);
+    if (res) {                                      // the residual add is taken along: out is the new residual row, rounded
+      acc += res[t * width + c];
+      res[t * width + c] = acc;
+    }
+    if (out) stf(out + t * width + c, acc);
   }
 }
 
@@ -525,14 +529,14 @@ extern "C" int nvs_moe_gemm(const void* X, int64_t ldx, const void* W, int dtype
 }
 
 extern "C" int nvs_moe_combine(const void* rows, int64_t ldr, const int32_t* pair_row, const float* wts, int top, const void* h, int64_t ldh,
-                               const void* shared, const float* shared_gate, int64_t gate_stride, int dtype, int64_t n, int width, void* out,
-                               void* stream) {
-  NVS_REQUIRE(rows && pair_row && wts && h && out && top > 0 && width > 0 && n >= 0,
+                               const void* shared, const float* shared_gate, int64_t gate_stride, int dtype, int64_t n, int width, float* res,
+                               void* out, void* stream) {
+  NVS_REQUIRE(rows && pair_row && wts && h && (out || res) && top > 0 && width > 0 && n >= 0,
               "nvs_moe_combine: bad argument");
   if (n == 0) return NVS_OK;
   const int threads = width >= 1024 ? 256 : (width >= 256 ? 128 : 64);
   NVS_DISPATCH(dtype, moe_combine_kernel<T><<<dim3((unsigned)n), dim3(threads), 0, (hipStream_t)stream>>>(
                           (const T*)rows, ldr, pair_row, wts, top, (const T*)h, ldh, (const T*)shared, shared_gate, gate_stride, width,
-                          (T*)out));
+                          res, (T*)out));
   return nvs_check_launch("nvs_moe_combine");
 }

@@ -20,7 +20,7 @@ int nvs_check_launch(const char* what) {
   }
   return NVS_OK;
 }
-extern "C" int nvs_abi_version(void) { return 5; }   // 5: norms on both sides of a sublayer, attention sinks and query temperature, the gated matrix memory, table-routed experts
+extern "C" int nvs_abi_version(void) { return 6; }   // 6: token-shift norms, gated lookups, the gated delta rule, pooled blocks behind an attention window, capped scores
 extern "C" const char* nvs_last_error(void) { return g_err; }
 
 namespace {
@@ -164,8 +164,8 @@ __global__ void add_group_norm_kernel(float* __restrict__ x, const T* __restrict
       ss = 0.f;
       for (int i = 0; i < wpg; ++i) ss += red[0][first * wpg + i];
     }
-    const float k = 1.f / sqrtf(ss / (float)gsz + eps);
-    for (int c = idx; c < gsz; c += stride) stf(out + r * width + c0 + c, (xr[c0 + c] - mean) * k * ldf(w + c0 + c));
+    const float k = w ? 1.f / sqrtf(ss / (float)gsz + eps) : 1.f;      // (no weights: the sum itself)
+    for (int c = idx; c < gsz; c += stride) stf(out + r * width + c0 + c, (xr[c0 + c] - mean) * k * (w ? ldf(w + c0 + c) : 1.f));
   }
 }
 
@@ -203,6 +203,118 @@ __global__ void sandwich_norm_kernel(float* __restrict__ x, const T* __restrict_
   }
   const float k = 1.f / sqrtf(block_sum(ss, red) / (float)width + eps);
   for (int c = threadIdx.x; c < width; c += blockDim.x) stf(out + r * width + c, xr[c] * k * (w_off + ldf(w + c)));
+}
+
+// x[t] = rms(table[ids[t]]) * w: one workgroup per token
+template <typename T>
+__global__ void embed_norm_kernel(const T* __restrict__ table, const int64_t* __restrict__ ids, int width, const T* __restrict__ w, float eps,
+                                  float* __restrict__ x) {
+  __shared__ float red[16];
+  const int64_t t = blockIdx.x;
+  const T* row = table + ids[t] * width;
+  float ss = 0.f;
+  for (int c = threadIdx.x; c < width; c += blockDim.x) {
+    const float v = ldf(row + c);
+    ss += v * v;
+  }
+  const float k = 1.f / sqrtf(block_sum(ss, red) / (float)width + eps);
+  for (int c = threadIdx.x; c < width; c += blockDim.x) x[t * width + c] = ldf(row + c) * k * ldf(w + c);
+}
+
+// The add, the norm and the blend with the previous token's normed row, in one pass. A workgroup takes `rows` consecutive token
+// rows and keeps the last normed row in LDS; ahead of its first row it norms the row before it once more (x is not updated in
+// place, so that row can still be read). The workgroup that holds a portion's FIRST row also norms its LAST one: it alone
+// reads and replaces the sequence's state. VEC columns per thread and access (4 where width allows).
+template <typename T, int VEC>
+__global__ __launch_bounds__(256) void shift_norm_kernel(const float* __restrict__ x, const T* __restrict__ a, const T* __restrict__ wa,
+                                                         const T* __restrict__ w, const T* __restrict__ mu, const int32_t* __restrict__ cu_q,
+                                                         const int32_t* __restrict__ ctx0, const int32_t* __restrict__ slot,
+                                                         const int32_t* __restrict__ tseq, int64_t n, int width, float eps, int rows,
+                                                         float* __restrict__ state, float* __restrict__ x_out, T* __restrict__ out) {
+  extern __shared__ __attribute__((aligned(16))) float shift_lds[];      // yrow | hrow: every thread only touches its own columns
+  __shared__ float red[16];
+  float *yrow = shift_lds, *hrow = shift_lds + width;
+  const int tid = threadIdx.x, step = blockDim.x * VEC;
+  // y of row t into yrow (and x_out); returns 1 / rms(y)
+  auto load = [&](int64_t t, bool store) {
+    float ka = 1.f;
+    if (a && wa) {
+      float ss = 0.f;
+      for (int c = tid * VEC; c < width; c += step) {
+        float v[VEC];
+        ldv<VEC>(a + t * width + c, v);
+#pragma unroll
+        for (int i = 0; i < VEC; ++i) ss += v[i] * v[i];
+      }
+      ka = 1.f / sqrtf(block_sum(ss, red) / (float)width + eps);
+    }
+    float ss = 0.f;
+    for (int c = tid * VEC; c < width; c += step) {
+      float y[VEC];
+      ldv<VEC>(x + t * width + c, y);
+      if (a) {
+        float v[VEC], g[VEC];
+        ldv<VEC>(a + t * width + c, v);
+        if (wa) ldv<VEC>(wa + c, g);
+#pragma unroll
+        for (int i = 0; i < VEC; ++i) y[i] += wa ? v[i] * ka * g[i] : v[i];
+        if (store) stv<VEC>(x_out + t * width + c, y);
+      }
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) ss += y[i] * y[i], yrow[c + i] = y[i];
+    }
+    return 1.f / sqrtf(block_sum(ss, red) / (float)width + eps);
+  };
+  const int64_t t0 = (int64_t)blockIdx.x * rows, t1 = t0 + rows < n ? t0 + rows : n;
+  for (int64_t t = t0; t < t1; ++t) {
+    const int s = tseq[t];
+    const int64_t q0 = cu_q[s], q1 = cu_q[s + 1];
+    float* st = state + (int64_t)slot[s] * width;
+    const bool head = t == q0, fresh = ctx0[s] == 0;
+    if (!head && t == t0) {                         // the row before the workgroup's first one
+      const float k = load(t - 1, false);
+      for (int c = tid * VEC; c < width; c += step) {
+        float g[VEC];
+        ldv<VEC>(w + c, g);
+#pragma unroll
+        for (int i = 0; i < VEC; ++i) hrow[c + i] = yrow[c + i] * k * g[i];
+      }
+    }
+    const float k = load(t, true);
+    for (int c = tid * VEC; c < width; c += step) {
+      float g[VEC], m[VEC], o[VEC];
+      ldv<VEC>(w + c, g);
+      ldv<VEC>(mu + c, m);
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) {
+        const float h = yrow[c + i] * k * g[i];
+        const float before = head ? (fresh ? 0.f : st[c + i]) : hrow[c + i];
+        o[i] = h + (before - h) * m[i];
+        hrow[c + i] = h;
+        if (head && q1 - q0 == 1) st[c + i] = h;
+      }
+      stv<VEC>(out + t * width + c, o);
+    }
+    if (head && q1 - q0 > 1) {                      // (hrow stays: the next row of this workgroup blends with it)
+      const float kl = load(q1 - 1, false);
+      for (int c = tid * VEC; c < width; c += step) {
+        float g[VEC];
+        ldv<VEC>(w + c, g);
+#pragma unroll
+        for (int i = 0; i < VEC; ++i) st[c + i] = yrow[c + i] * kl * g[i];
+      }
+    }
+  }
+}
+
+template <typename T>
+__global__ void gated_lookup_kernel(const T* __restrict__ z, int64_t z_stride, const T* __restrict__ table, int64_t table_stride, int64_t col0,
+                                    const int64_t* __restrict__ ids, int dim, int64_t total, T* __restrict__ out) {
+  for (int64_t i = (int64_t)blockIdx.x * blockDim.x + threadIdx.x; i < total; i += (int64_t)gridDim.x * blockDim.x) {
+    const int64_t t = i / dim;
+    const int c = (int)(i - t * dim);
+    stf(out + i, gelu_tanhf_(ldf(z + t * z_stride + c)) * ldf(table + ids[t] * table_stride + col0 + c));
+  }
 }
 
 // logits <- cap * tanh(logits * scale / cap) (cap <= 0: logits * scale), 32-bit out
@@ -257,7 +369,7 @@ extern "C" int nvs_xielu(const void* in, const void* pq, float beta, int dtype, 
 
 extern "C" int nvs_add_group_norm(float* x, const void* a, float a_mult, const float* b, const int32_t* rows, int64_t nrows, const void* w,
                                   int dtype, int width, int groups, float eps, int center, void* out, void* stream) {
-  NVS_REQUIRE(x && nrows >= 0 && width > 0 && groups > 0 && width % groups == 0 && (!out || w), "nvs_add_group_norm: width %d groups %d",
+  NVS_REQUIRE(x && nrows >= 0 && width > 0 && groups > 0 && width % groups == 0 && (!out || w || !center), "nvs_add_group_norm: width %d groups %d",
               width, groups);
   NVS_REQUIRE(!rows || (!a && !b), "nvs_add_group_norm: selected rows are only read");
   if (nrows == 0) return NVS_OK;
@@ -286,4 +398,52 @@ extern "C" int nvs_scale_softcap(const void* in, int dtype, float scale, float c
   NVS_DISPATCH(dtype, scale_softcap_kernel<T><<<dim3((unsigned)(blocks > 65536 ? 65536 : blocks)), dim3(256), 0, (hipStream_t)stream>>>(
                           (const T*)in, scale, cap, numel, out));
   return nvs_check_launch("nvs_scale_softcap");
+}
+
+extern "C" int nvs_embed_norm(const void* table, int dtype, const int64_t* ids, int64_t n, int width, const void* w, float eps, float* x,
+                              void* stream) {
+  NVS_REQUIRE(table && ids && w && x && n >= 0 && width > 0, "nvs_embed_norm: bad argument (width %d)", width);
+  if (n == 0) return NVS_OK;
+  NVS_DISPATCH(dtype, embed_norm_kernel<T><<<dim3((unsigned)n), dim3(threads_for(width)), 0, (hipStream_t)stream>>>(
+                          (const T*)table, ids, width, (const T*)w, eps, x));
+  return nvs_check_launch("nvs_embed_norm");
+}
+
+extern "C" int nvs_shift_norm(const float* x, const void* a, const void* wa, const void* w, const void* mu, int dtype, const int32_t* cu_q,
+                              const int32_t* ctx0, const int32_t* slot, const int32_t* tseq, int nseq, int64_t n, int width, float eps,
+                              float* state, float* x_out, void* out, void* stream) {
+  NVS_REQUIRE(x && w && mu && cu_q && ctx0 && slot && tseq && state && out && n >= 0 && nseq >= 0, "nvs_shift_norm: null argument");
+  NVS_REQUIRE(width > 0 && width <= 16384, "nvs_shift_norm: width %d (up to 16384)", width);
+  NVS_REQUIRE(!wa || a, "nvs_shift_norm: a norm weight without a branch");
+  NVS_REQUIRE(!a || (x_out && x_out != x), "nvs_shift_norm: the sum needs a tensor of its own (rows of x are read twice)");
+  if (n == 0 || nseq == 0) return NVS_OK;
+  const int rows = n >= 8192 ? 8 : (n >= 2048 ? 4 : 1);       // (a workgroup reads one row more than it writes)
+  const size_t lds = 2 * (size_t)width * sizeof(float);
+  const dim3 grid((unsigned)((n + rows - 1) / rows)), block(width >= 1024 ? 256 : (width >= 256 ? 128 : 64));
+#define NVS_SHIFT(VEC)                                                                                                                  \
+  NVS_DISPATCH(dtype, {                                                                                                                 \
+    if (lds > 48 * 1024)                                                                                                                \
+      (void)hipFuncSetAttribute((const void*)shift_norm_kernel<T, VEC>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);           \
+    shift_norm_kernel<T, VEC><<<grid, block, lds, (hipStream_t)stream>>>(x, (const T*)a, (const T*)wa, (const T*)w, (const T*)mu, cu_q, ctx0, \
+                                                                         slot, tseq, n, width, eps, rows, state, x_out, (T*)out);        \
+  })
+  if (width % 4 == 0) {
+    NVS_SHIFT(4);
+  } else {
+    NVS_SHIFT(1);
+  }
+#undef NVS_SHIFT
+  return nvs_check_launch("nvs_shift_norm");
+}
+
+extern "C" int nvs_gated_lookup(const void* z, int64_t z_stride, const void* table, int64_t table_stride, int64_t col0, int dtype,
+                                const int64_t* ids, int dim, int64_t n, void* out, void* stream) {
+  NVS_REQUIRE(z && table && ids && out && dim > 0 && n >= 0 && z_stride >= dim && col0 >= 0 && table_stride >= col0 + dim,
+              "nvs_gated_lookup: %d columns from %lld on of rows of %lld", dim, (long long)col0, (long long)table_stride);
+  if (n == 0) return NVS_OK;
+  int64_t blocks = (n * dim + 255) / 256;
+  if (blocks > 65535) blocks = 65535;
+  NVS_DISPATCH(dtype, gated_lookup_kernel<T><<<dim3((unsigned)blocks), dim3(256), 0, (hipStream_t)stream>>>(
+                          (const T*)z, z_stride, (const T*)table, table_stride, col0, ids, dim, n * dim, (T*)out));
+  return nvs_check_launch("nvs_gated_lookup");
 }

@@ -43,6 +43,41 @@ __global__ void causal_conv_kernel(const T* __restrict__ in, int64_t in_stride, 
   stf(out + t * channels + c, acc);
 }
 
+// Steps of short portions (decoding): one thread per (portion, channel) walks the portion's tokens with the last taps - 1 inputs in
+// registers and leaves them in the slot — outputs and state in one launch.
+template <typename T, typename TO, int TAPS>
+__global__ void conv_walk_kernel(const T* __restrict__ in, int64_t in_stride, const T* __restrict__ w, const T* __restrict__ b, int channels,
+                                 int act, const int32_t* __restrict__ cu_q, const int32_t* __restrict__ ctx0, const int32_t* __restrict__ slot,
+                                 float* __restrict__ state, TO* __restrict__ out) {
+  const int s = blockIdx.y;
+  const int c = blockIdx.x * blockDim.x + threadIdx.x;
+  if (c >= channels) return;
+  const int64_t q0 = cu_q[s], q1 = cu_q[s + 1];
+  if (q1 <= q0) return;
+  float* tail = state + (int64_t)slot[s] * (TAPS - 1) * channels + c;
+  const bool fresh = ctx0[s] == 0;
+  float past[TAPS - 1], wt[TAPS];
+#pragma unroll
+  for (int k = 0; k < TAPS - 1; ++k) past[k] = fresh ? 0.f : tail[(int64_t)k * channels];
+#pragma unroll
+  for (int k = 0; k < TAPS; ++k) wt[k] = ldf(w + (int64_t)c * TAPS + k);
+  const float bias = b ? ldf(b + c) : 0.f;
+  for (int64_t t = q0; t < q1; ++t) {
+    const float v = ldf(in + t * in_stride + c);
+    float acc = bias;
+#pragma unroll
+    for (int k = 0; k < TAPS - 1; ++k) acc += wt[k] * past[k];
+    acc += wt[TAPS - 1] * v;
+#pragma unroll
+    for (int k = 0; k + 1 < TAPS - 1; ++k) past[k] = past[k + 1];
+    past[TAPS - 2] = v;
+    if (act == 1) acc = siluf_(acc);
+    stf(out + t * channels + c, acc);
+  }
+#pragma unroll
+  for (int k = 0; k < TAPS - 1; ++k) tail[(int64_t)k * channels] = past[k];
+}
+
 // one thread per (portion, channel): the new tail is read completely before it is written
 template <typename T>
 __global__ void conv_state_kernel(const T* __restrict__ in, int64_t in_stride, int channels, int taps,
@@ -483,13 +518,14 @@ __global__ __launch_bounds__(FORM == 2 ? (PP == 4 ? 512 : (PP == 2 ? 576 : 1024)
 // one workgroup per (token, group)
 template <typename T>
 __global__ void gated_group_norm_kernel(const float* __restrict__ y, const T* __restrict__ z, int64_t z_stride,
-                                        const T* __restrict__ w, int inner, int groups, float eps, int order,
+                                        const T* __restrict__ w, int wlen, int inner, int groups, float eps, int order,
                                         const float* __restrict__ den, T* __restrict__ out) {
   __shared__ float red[16];
   const int64_t t = blockIdx.y;
   const int gsz = inner / groups, c0 = blockIdx.x * gsz;
   float ss = 0.f;
-  if (order == 1) {                                 // norm first, then a sigmoid gate
+  if (wlen < inner) w -= c0;                        // one set of weights for all groups
+  if (order >= 1) {                                 // norm first, then a sigmoid (or SiLU) gate
     const float dinv = den ? 1.f / den[t * groups + blockIdx.x] : 1.f;      // the group's entries are numerators over this
     for (int c = threadIdx.x; c < gsz; c += blockDim.x) {
       const float v = y[t * inner + c0 + c] * dinv;
@@ -498,7 +534,7 @@ __global__ void gated_group_norm_kernel(const float* __restrict__ y, const T* __
     const float r = 1.f / sqrtf(block_sum(ss, red) / (float)gsz + eps);
     for (int c = threadIdx.x; c < gsz; c += blockDim.x) {
       const float gz = ldf(z + t * z_stride + c0 + c);
-      stf(out + t * inner + c0 + c, y[t * inner + c0 + c] * dinv * r * ldf(w + c0 + c) * (1.f / (1.f + expf(-gz))));
+      stf(out + t * inner + c0 + c, y[t * inner + c0 + c] * dinv * r * ldf(w + c0 + c) * ((order == 2 ? gz : 1.f) / (1.f + expf(-gz))));
     }
     return;
   }
@@ -526,6 +562,22 @@ extern "C" int nvs_causal_conv(const void* in, int64_t in_stride, int dtype, con
   NVS_REQUIRE(n <= 65535 * 64ll && nseq <= 65535, "nvs_causal_conv: step too large");
   const dim3 block(channels >= 256 ? 256 : 64);
   const unsigned gx = (channels + block.x - 1) / block.x;
+  if (taps >= 2 && taps <= 4 && n <= 4ll * nseq) {
+#define NVS_CONV_WALK(TAPS)                                                                                                            \
+  do {                                                                                                                                 \
+    if (out_dtype == NVS_F32)                                                                                                          \
+      NVS_DISPATCH(dtype, conv_walk_kernel<T, float, TAPS><<<dim3(gx, (unsigned)nseq), block, 0, (hipStream_t)stream>>>(                \
+                              (const T*)in, in_stride, (const T*)w, (const T*)b, channels, act, cu_q, ctx0, slot, state, (float*)out)); \
+    else                                                                                                                               \
+      NVS_DISPATCH(dtype, conv_walk_kernel<T, T, TAPS><<<dim3(gx, (unsigned)nseq), block, 0, (hipStream_t)stream>>>(                    \
+                              (const T*)in, in_stride, (const T*)w, (const T*)b, channels, act, cu_q, ctx0, slot, state, (T*)out));     \
+  } while (0)
+    if (taps == 2) NVS_CONV_WALK(2);
+    else if (taps == 3) NVS_CONV_WALK(3);
+    else NVS_CONV_WALK(4);
+#undef NVS_CONV_WALK
+    return nvs_check_launch("nvs_causal_conv (short portions)");
+  }
   // grid.y is limited to 65535: larger steps go in slices
   for (int64_t t0 = 0; t0 < n; t0 += 65535) {
     const int64_t cnt = n - t0 < 65535 ? n - t0 : 65535;
@@ -716,11 +768,11 @@ extern "C" int nvs_gated_memory_scan(const void* proj, int64_t proj_stride, int6
                     heads, dv + 1, dk, heads, cu_q, ctx0, slot, nseq, n, max_q, S, y, ws, ws_floats, stream, ga);
 }
 
-extern "C" int nvs_gated_group_norm(const float* y, const void* z, int64_t z_stride, int dtype, const void* w, int inner, int groups,
+extern "C" int nvs_gated_group_norm(const float* y, const void* z, int64_t z_stride, int dtype, const void* w, int wlen, int inner, int groups,
                                     float eps, int order, int64_t n, const float* den, void* out, void* stream) {
-  NVS_REQUIRE(!den || order == 1, "nvs_gated_group_norm: a divisor goes with the order norm, then gate");
+  NVS_REQUIRE(!den || order >= 1, "nvs_gated_group_norm: a divisor goes with the order norm, then gate");
   NVS_REQUIRE(y && z && w && out && inner > 0 && groups > 0 && inner % groups == 0 && z_stride >= inner && n >= 0 &&
-                  (order == 0 || order == 1),
+                  order >= 0 && order <= 2 && (wlen == inner || wlen * groups == inner),
               "nvs_gated_group_norm: inner %d groups %d order %d", inner, groups, order);
   if (n == 0) return NVS_OK;
   NVS_REQUIRE(n <= 65535ll * 65535ll, "nvs_gated_group_norm: step too large");
@@ -729,7 +781,7 @@ extern "C" int nvs_gated_group_norm(const float* y, const void* z, int64_t z_str
   for (int64_t t0 = 0; t0 < n; t0 += 65535) {
     const int64_t cnt = n - t0 < 65535 ? n - t0 : 65535;
     NVS_DISPATCH(dtype, gated_group_norm_kernel<T><<<dim3(groups, (unsigned)cnt), block, 0, (hipStream_t)stream>>>(
-                            y + t0 * inner, (const T*)z + t0 * z_stride, z_stride, (const T*)w, inner, groups, eps, order,
+                            y + t0 * inner, (const T*)z + t0 * z_stride, z_stride, (const T*)w, wlen, inner, groups, eps, order,
                             den ? den + t0 * groups : nullptr, (T*)out + t0 * inner));
   }
   return nvs_check_launch("nvs_gated_group_norm");

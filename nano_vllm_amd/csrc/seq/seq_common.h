@@ -25,6 +25,51 @@ __device__ __forceinline__ float ldf(const bf16_t* p) { return (float)*p; }
 __device__ __forceinline__ void stf(float* p, float v) { *p = v; }
 __device__ __forceinline__ void stf(bf16_t* p, float v) { *p = (bf16_t)v; }   // round to nearest even
 
+// VEC consecutive elements at once (16 / 8 bytes for VEC 4; the address is aligned to VEC elements)
+template <int VEC>
+__device__ __forceinline__ void ldv(const float* p, float (&v)[VEC]) {
+  if constexpr (VEC == 4) {
+    const float4 f = *(const float4*)p;
+    v[0] = f.x, v[1] = f.y, v[2] = f.z, v[3] = f.w;
+  } else {
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) v[i] = p[i];
+  }
+}
+template <int VEC>
+__device__ __forceinline__ void ldv(const bf16_t* p, float (&v)[VEC]) {
+  if constexpr (VEC == 4) {
+    typedef __attribute__((ext_vector_type(4))) __bf16 b4_t;
+    const b4_t b = *(const b4_t*)p;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) v[i] = (float)b[i];
+  } else {
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) v[i] = (float)p[i];
+  }
+}
+template <int VEC>
+__device__ __forceinline__ void stv(float* p, const float (&v)[VEC]) {
+  if constexpr (VEC == 4) *(float4*)p = make_float4(v[0], v[1], v[2], v[3]);
+  else {
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) p[i] = v[i];
+  }
+}
+template <int VEC>
+__device__ __forceinline__ void stv(bf16_t* p, const float (&v)[VEC]) {
+  if constexpr (VEC == 4) {
+    typedef __attribute__((ext_vector_type(4))) __bf16 b4_t;
+    b4_t b;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) b[i] = (bf16_t)v[i];
+    *(b4_t*)p = b;
+  } else {
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) p[i] = (bf16_t)v[i];
+  }
+}
+
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll
   for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);

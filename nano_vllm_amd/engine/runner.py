@@ -895,7 +895,10 @@ class ModelRunner:
         st_layers = [m for m in self.model.modules() if hasattr(m, "state_shapes")]
         esize = torch.finfo(self.dtype).bits // 8
         per_token = sum(int(np.prod(k)) + int(np.prod(v)) for k, v in (m.kv_shapes() for m in kv_layers)) * esize
-        block_bytes = max(per_token * self.block_size, 1)
+        # tensors with rows per PAGE (summaries of the page's tokens): they come and go with the pages
+        page_layers = [m for m in self.model.modules() if hasattr(m, "page_shapes")]
+        per_page = sum(int(np.prod(shape)) for m in page_layers for shape in m.page_shapes().values()) * esize
+        block_bytes = max(per_token * self.block_size + per_page, 1)
         for m in st_layers:                                       # state first: small, and it is not optional
             for name, shape in m.state_shapes().items():
                 # (one slot more than sequences: the scratch slot of a captured decode step's padding rows)
@@ -916,6 +919,9 @@ class ModelRunner:
             m.k_cache = torch.zeros(slots, *ks, dtype=self.dtype, device=self.device)
             m.v_cache = torch.zeros(slots, *vs, dtype=self.dtype, device=self.device)
             m.block_size = self.block_size
+        for m in page_layers:
+            for name, shape in m.page_shapes().items():
+                setattr(m, name, torch.zeros(cfg.num_kvcache_blocks, *shape, dtype=self.dtype, device=self.device))
 
     def prepare_portions(self, seqs: list[Sequence], want: list[list[int]] | None = None, pad_to: int = 0) -> dict:
         """Fill the staging block for a packed step: sequence i contributes tokens [num_cached_tokens, + num_scheduled_tokens).

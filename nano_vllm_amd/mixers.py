@@ -2,8 +2,9 @@
 
   WindowAttention     paged softmax attention with a local mask (a sliding window, or blocks of positions, or none), any
                       query / value head size, optional per-head q/k RMS norm, optional rotation of the leading dimensions
-                      in interleaved pairs, optional sigmoid output gate
-  AttentionMixer      fused biased q | k | v projection -> WindowAttention -> out projection
+                      in interleaved pairs, optional sigmoid output gate, capped scores, a norm over the whole query / key
+                      projection, means over blocks of positions behind the window, another layer's keys and values
+  AttentionMixer      fused q | k | v projection (biased or not) -> WindowAttention -> out projection
   ConvAttentionMixer  attention whose query and key projections pass a short stateful causal convolution, whose keys (before
                       rotation) are also its values, with a constant or learned sink in the softmax and a gate per head
   GatedMemoryCore     matrix memory with exponential input / forget gates held in range by a running maximum (mLSTM style),
@@ -14,6 +15,11 @@
                       shared by the heads; runs in the latent space on WindowAttention's kernels (one kv head), with a query
                       latent, either rotary pairing, optional frequency scaling, window or causal mask, optional per-head
                       sigmoid gate, and optionally the cache of an earlier layer instead of its own
+  DeltaMixer          gated delta rule (the write is the error of the state's answer for the key): stateful convolution + SiLU on
+                      q / k / v, unit vectors, a decay per head or per head and key channel, norm per head, SiLU or low-rank
+                      sigmoid gate
+  TokenShiftNorm      pre-norm whose output is blended with the previous token's, channel by channel
+  TokenSide           a branch that multiplies a gate of the residual with a second embedding of the token
   LightningMixer      linear attention as a decaying outer-product recurrence (per-head constant decay), SiLU on q / k / v,
                       RMS norm over the heads together, sigmoid gate
   SSDMixer            state-space-duality (Mamba-2 style) mixer: stateful causal convolution + SiLU, the recurrence in
@@ -62,8 +68,13 @@ class WindowAttention(nn.Module):
 
     def __init__(self, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, window: int, eps: float,
                  qk_norm: bool = True, block_size: int = 256, chunk: int = 0, rot_dims: int = 0, rot_base: float = 10000.0,
-                 rot_freqs: list | None = None, sink: str | None = None, q_temp: tuple | None = None, gate_per_head: bool = False):
-        """window > 0: the last `window` positions are visible; chunk > 0: the positions of the query's own block of `chunk`
+                 rot_freqs: list | None = None, sink: str | None = None, q_temp: tuple | None = None, gate_per_head: bool = False,
+                 norm_rows: bool = False, softcap: float = 0.0, pool: int = 0, source: "WindowAttention | None" = None):
+        """norm_rows: the query and key norms are over the whole projection (all heads together), not per head. softcap > 0: scores
+        become softcap tanh(score / softcap). pool > 0 (behind a window): beside the window's tokens a query sees the mean key and
+        value of every block of `pool` positions that lies wholly before it. source: an earlier layer's attention whose cached
+        keys and values this one reads instead of keeping its own (its k and v are then None).
+        window > 0: the last `window` positions are visible; chunk > 0: the positions of the query's own block of `chunk`
         (counted from the start of the sequence); neither: all earlier positions. rot_dims > 0: entries (2i, 2i+1),
         i < rot_dims / 2, of every query and key head turn by position * rot_base^(-2i / rot_dims), or by position * rot_freqs[i]
         when the caller brings its own table of rot_dims / 2 frequencies. sink: "zero" puts one more score of 0 (no value) into every
@@ -76,7 +87,13 @@ class WindowAttention(nn.Module):
             self.sink = _param(heads, dtype=torch.float32)
         else:
             self.register_buffer("sink", torch.zeros(heads, dtype=torch.float32) if sink else None, persistent=False)
-        assert heads % kv_heads == 0 and dim <= 256 and vdim <= 256 and not (window > 0 and chunk > 0)
+        assert heads % kv_heads == 0 and dim <= 1024 and vdim <= 1024 and not (window > 0 and chunk > 0)
+        self.norm_rows, self.softcap, self.pool = bool(norm_rows), float(softcap or 0.0), int(pool)
+        assert not self.pool or window > 0
+        self._source = (source,) if source is not None else ()          # (a tuple: not a submodule of this layer)
+        if source is not None:
+            assert not source._source and (source.G, source.d, source.dv) == (kv_heads, dim, vdim), "the borrowed cache has other sizes, or is borrowed itself"
+        self.pool_k = self.pool_v = None              # [pages, rows, G, d] / [pages, rows / 8, G, dv, 8], from the runner
         assert rot_dims % 2 == 0 and 0 <= rot_dims <= dim
         self.H, self.G, self.d, self.dv = heads, kv_heads, dim, vdim
         self.scale, self.window, self.eps, self.block_size = float(scale), int(window), eps, block_size
@@ -84,8 +101,8 @@ class WindowAttention(nn.Module):
         # frequencies in double precision on the host, rounded once; angles are position * frequency in 32-bit
         freqs = rot_freqs if rot_freqs is not None else [float(rot_base) ** (-2.0 * i / rot_dims) for i in range(rot_dims // 2)]
         self.register_buffer("rot_freq", torch.tensor(freqs, dtype=torch.float32) if rot_dims else None, persistent=False)
-        self.q_norm = _param(dim) if qk_norm else None
-        self.k_norm = _param(dim) if qk_norm else None
+        self.q_norm = _param(heads * dim if norm_rows else dim) if qk_norm else None
+        self.k_norm = _param(kv_heads * dim if norm_rows else dim) if qk_norm and source is None else None
         self.k_cache = self.v_cache = None            # [pages * block_size, G, d] / [..., G, dv] (values page-transposed), from the runner
 
     @property
@@ -94,43 +111,82 @@ class WindowAttention(nn.Module):
         return self.H * self.d, self.G * self.d, self.G * self.dv, self.H * self.dv
 
     def kv_shapes(self) -> tuple[tuple, tuple]:
-        """Per-token shapes of this layer's K and V pages."""
-        return (self.G, self.d), (self.G, self.dv)
+        """Per-token shapes of this layer's K and V pages (None: it reads another layer's)."""
+        return None if self._source else ((self.G, self.d), (self.G, self.dv))
+
+    @property
+    def owner(self) -> "WindowAttention":
+        """The layer whose keys and values this one reads."""
+        return self._source[0] if self._source else self
+
+    @property
+    def _own_pool(self) -> bool:
+        """Means over blocks of the owner's length are the owner's; a borrower with another block length keeps its own."""
+        return self.pool > 0 and (not self._source or self._source[0].pool != self.pool)
+
+    def page_shapes(self) -> dict:
+        """Per-page tensors beside K and V: the means over blocks of positions that end in a page."""
+        if not self._own_pool:
+            return {}
+        rows = ops_seq.pool_rows(self.block_size, self.pool)
+        return {"pool_k": (rows, self.G, self.d), "pool_v": (rows // 8, self.G, self.dv, 8)}
 
     def forward(self, q, k, v, gate, positions: torch.Tensor | None = None) -> torch.Tensor:
         ctx = get_context()
-        ops_seq.knorm_kvstore(k, v, self.k_norm, self.eps, self.G, self.d, self.dv, self.block_size, ctx.slot_mapping, self.k_cache,
-                              self.v_cache, positions, self.rot_freq)
+        own, q_row = self.owner, None
+        means = self if self._own_pool else own
+        if self.norm_rows:
+            q_row = ops_seq.qk_rows(q, k, v, self.k_norm, self.eps, self.G, self.d, self.dv, self.block_size, ctx.slot_mapping, own.k_cache,
+                                    own.v_cache, positions, self.rot_freq, ctx.portions, ctx.block_tables, self.pool, means.pool_k, means.pool_v)
+        elif k is not None:
+            ops_seq.knorm_kvstore(k, v, self.k_norm, self.eps, self.G, self.d, self.dv, self.block_size, ctx.slot_mapping, own.k_cache,
+                                  own.v_cache, positions, self.rot_freq)
+        if self._own_pool and (k is None or not self.norm_rows):
+            ops_seq.pool_blocks(own.k_cache, own.v_cache, self.G, self.d, self.dv, self.block_size, self.pool, ctx.slot_mapping, positions,
+                                ctx.block_tables, ctx.portions, self.pool_k, self.pool_v)
         out = torch.empty(q.shape[0], self.H * self.dv, dtype=q.dtype, device=q.device)
-        ops_seq.window_attn(q, self.q_norm, self.eps, gate, self.k_cache, self.v_cache, ctx.block_tables, self.block_size,
+        ops_seq.window_attn(q, self.q_norm, self.eps, gate, own.k_cache, own.v_cache, ctx.block_tables, self.block_size,
                             ctx.portions, self.H, self.G, self.d, self.dv, self.scale, self.window, out, self.chunk, self.rot_freq,
-                            gate_per_head=self.gate_per_head, sink=self.sink, q_temp=self.q_temp)
+                            gate_per_head=self.gate_per_head, sink=self.sink, q_temp=self.q_temp, q_row=q_row, softcap=self.softcap,
+                            pool=self.pool, pool_k=means.pool_k, pool_v=means.pool_v)
         return out
 
 
 class AttentionMixer(nn.Module):
-    """q | k | v in ONE biased projection, attention (WindowAttention: mask, rotation), out projection."""
+    """q | k | v in ONE projection (with `bias`, biased), attention (WindowAttention: mask, rotation and its other options), out
+    projection. source: an earlier layer's AttentionMixer whose keys and values are read; there is then no k | v projection."""
 
     def __init__(self, width: int, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, eps: float, block_size: int,
-                 window: int = 0, chunk: int = 0, rot_dims: int = 0, rot_base: float = 10000.0, qk_norm: bool = False):
+                 window: int = 0, chunk: int = 0, rot_dims: int = 0, rot_base: float = 10000.0, qk_norm: bool = False, bias: bool = True,
+                 source: "AttentionMixer | None" = None, **options):
         super().__init__()
         self.attn = WindowAttention(heads, kv_heads, dim, vdim, scale, window, eps, qk_norm=qk_norm, block_size=block_size,
-                                    chunk=chunk, rot_dims=rot_dims, rot_base=rot_base)
-        self.cols = self.attn.widths[:3]
+                                    chunk=chunk, rot_dims=rot_dims, rot_base=rot_base, source=source.attn if source is not None else None, **options)
+        self.cols = self.attn.widths[:3] if source is None else (self.attn.widths[0], 0, 0)
         total = sum(self.cols)
-        self.in_w, self.in_b = _param(total, width), _param(total)
+        self.in_w, self.in_b = _param(total, width), _param(total) if bias else None
         self.o_w = _param(width, heads * vdim)
 
     def named_loaders(self) -> dict:
-        q, k, v = self.cols
-        return {"q": _copy_into(self.in_w[:q]), "q.b": _copy_into(self.in_b[:q]), "k": _copy_into(self.in_w[q:q + k]),
-                "k.b": _copy_into(self.in_b[q:q + k]), "v": _copy_into(self.in_w[q + k:]), "v.b": _copy_into(self.in_b[q + k:]),
-                "o": _copy_into(self.o_w)}
+        out, at = {"o": _copy_into(self.o_w)}, 0
+        for name, cols in zip("qkv", self.cols):
+            if cols:
+                out[name] = _copy_into(self.in_w[at:at + cols])
+                if self.in_b is not None:
+                    out[name + ".b"] = _copy_into(self.in_b[at:at + cols])
+            at += cols
+        for name, w in (("q.norm", self.attn.q_norm), ("k.norm", self.attn.k_norm)):
+            if w is not None:
+                out[name] = _copy_into(w)
+        if isinstance(self.attn.sink, nn.Parameter):
+            out["sink"] = _copy_into(self.attn.sink)
+        return out
 
     def forward(self, xh: torch.Tensor, positions: torch.Tensor) -> torch.Tensor:
         proj = F.linear(xh, self.in_w, self.in_b)
-        q, k, v = self.cols
-        return F.linear(self.attn(proj[:, :q], proj[:, q:q + k], proj[:, q + k:], None, positions), self.o_w)
+        q, k, _ = self.cols
+        kv = (proj[:, q:q + k], proj[:, q + k:]) if k else (None, None)
+        return F.linear(self.attn(proj[:, :q], *kv, None, positions), self.o_w)
 
 
 def rotary_frequencies(dims: int, base: float, scaling: dict | None = None) -> tuple[list[float], float]:
@@ -361,6 +417,102 @@ class LatentAttentionMixer(nn.Module):
         return F.linear(out.view(n, H * dv), self.o_w)
 
 
+class DeltaMixer(nn.Module):
+    """The gated delta rule. q, k (kv_heads of `dim`) and v (heads of `vdim`) pass a short stateful causal convolution and SiLU;
+    q and k become unit vectors per head, q times dim^(-1/2); with a step size beta = sigmoid(W_b h) and a decay g per head,
+        S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q          (state and everything on this line in 32-bit),
+    g = exp(-exp(A_log) softplus(W_a h + dt_bias)) — or, with decay_rank > 0, one per head and KEY CHANNEL, from W_a2 (W_a1 h).
+    Every head's o is divided by its root mean square, times `norm` (one set of vdim weights), times silu(W_g h) — or, with
+    gate_rank > 0, sigmoid(W_g2 (W_g1 h)) — and projected. ONE in-projection [q | k | v | g or g1 | a or a1 | b]."""
+
+    def __init__(self, width: int, heads: int, kv_heads: int, dim: int, vdim: int, taps: int, eps: float, decay_rank: int = 0, gate_rank: int = 0):
+        super().__init__()
+        assert heads % kv_heads == 0 and taps >= 1
+        self.H, self.G, self.d, self.dv, self.taps, self.eps = heads, kv_heads, dim, vdim, int(taps), eps
+        self.a_rank, self.g_rank = int(decay_rank), int(gate_rank)
+        self.channels = 2 * kv_heads * dim + heads * vdim
+        self.cols = (kv_heads * dim, kv_heads * dim, heads * vdim, self.g_rank or heads * vdim, self.a_rank or heads, heads)
+        self.in_w = _param(sum(self.cols), width)
+        self.conv_w = _param(self.channels, taps)
+        self.a2 = _param(heads * dim, self.a_rank) if self.a_rank else None
+        self.g2 = _param(heads * vdim, self.g_rank) if self.g_rank else None
+        self.A_log = _param(heads, dtype=torch.float32)
+        self.dt_bias = _param(heads * dim if self.a_rank else heads, dtype=torch.float32)
+        self.norm = _param(vdim)
+        self.o_w = _param(width, heads * vdim)
+        self.conv_state = self.rec_state = None
+
+    def state_shapes(self) -> dict:
+        return {"conv_state": (self.taps - 1, self.channels), "rec_state": (self.H, self.dv, self.d)}
+
+    def named_loaders(self) -> dict:
+        names = ("q", "k", "v", "g1" if self.g_rank else "g", "a1" if self.a_rank else "a", "b")
+        out, at = {}, 0
+        for i, (name, cols) in enumerate(zip(names, self.cols)):
+            out[name] = _copy_into(self.in_w[at:at + cols])
+            if i < 3:
+                out[name + ".conv"] = _copy_into(self.conv_w[at:at + cols])
+            at += cols
+        out.update({"A_log": _copy_into(self.A_log), "dt_bias": _copy_into(self.dt_bias), "norm": _copy_into(self.norm), "o": _copy_into(self.o_w)})
+        if self.a_rank:
+            out["a2"] = _copy_into(self.a2)
+        if self.g_rank:
+            out["g2"] = _copy_into(self.g2)
+        return out
+
+    def forward(self, xh: torch.Tensor, positions: torch.Tensor | None = None) -> torch.Tensor:
+        por = get_context().portions
+        n, c = xh.shape[0], self.channels
+        proj = F.linear(xh, self.in_w)
+        g_col, a_col = c, c + self.cols[3]
+        b_col = a_col + self.cols[4]
+        qkv = torch.empty(n, c, dtype=xh.dtype, device=xh.device)
+        ops_seq.causal_conv(proj[:, :c], self.conv_w, None, 1, por, self.conv_state, qkv)
+        decays = F.linear(proj[:, a_col:b_col], self.a2) if self.a_rank else None
+        gate = F.linear(proj[:, g_col:a_col], self.g2) if self.g_rank else proj[:, g_col:a_col]
+        y = torch.empty(n, self.H * self.dv, dtype=torch.float32, device=xh.device)
+        ops_seq.delta_scan(qkv, proj, b_col, 0 if self.a_rank else a_col, decays, self.A_log, self.dt_bias, self.d ** -0.5, self.H, self.G,
+                           self.d, self.dv, por, self.rec_state, y)
+        out = torch.empty(n, self.H * self.dv, dtype=xh.dtype, device=xh.device)
+        ops_seq.gated_group_norm(y, gate, self.norm, self.H, self.eps, out, norm_first=True, silu=not self.g_rank)
+        return F.linear(out, self.o_w)
+
+
+class TokenShiftNorm(nn.Module):
+    """Pre-norm with a token shift: h = rms(x) * w, the output h + (h of the previous token - h) * shift; the previous token's h is
+    per-sequence state. The add that comes before the norm (a branch, as it is or RMS-normed with weights) is taken along."""
+
+    def __init__(self, width: int, eps: float):
+        super().__init__()
+        self.width, self.eps = width, eps
+        self.w, self.shift = _param(width), _param(width)
+        self.shift_state = None
+
+    def state_shapes(self) -> dict:
+        return {"shift_state": (self.width,)}
+
+    def forward(self, x: torch.Tensor, a: torch.Tensor | None, wa: torch.Tensor | None, dtype) -> tuple[torch.Tensor, torch.Tensor]:
+        """(x with the branch added, the shifted normed row)."""
+        h = torch.empty(x.shape, dtype=dtype, device=x.device)
+        return ops_seq.shift_norm(x, a, wa, self.w, self.shift, self.eps, get_context().portions, self.shift_state, h), h
+
+
+class TokenSide(nn.Module):
+    """A branch that reads the token again: W_proj (gelu(W_gate x) * e), e = columns [col0, col0 + dim) of the token's row in a
+    second embedding table. Returns the branch before its norm; the kernel that adds it norms it with `norm`."""
+
+    def __init__(self, width: int, dim: int, col0: int):
+        super().__init__()
+        self.col0 = col0
+        self.gate, self.proj, self.norm = _param(dim, width), _param(width, dim), _param(width)
+
+    def named_loaders(self) -> dict:
+        return {"gate": _copy_into(self.gate), "proj": _copy_into(self.proj), "norm": _copy_into(self.norm)}
+
+    def forward(self, xh: torch.Tensor, table: torch.Tensor, ids: torch.Tensor) -> torch.Tensor:
+        return F.linear(ops_seq.gated_lookup(F.linear(xh, self.gate), table, self.col0, ids), self.proj)
+
+
 class LightningMixer(nn.Module):
     """Linear attention in its recurrent form: q, k, v = SiLU of the projections; per head S <- decay_h S + k v^T, o = S^T q
     (state and products in 32-bit); the heads together are RMS-normed (weight `norm`), multiplied by sigmoid(W_g h) and
@@ -587,11 +739,12 @@ class RoutedExperts(nn.Module):
 
     def __init__(self, width: int, experts: int, ff: int, top: int, scale: float = 1.0, identity: int = 0, group_count: int = 1,
                  group_keep: int = 1, shared_ff: int = 0, gated: bool = True, sigmoid: bool = False, renorm: bool = True,
-                 table_vocab: int = 0, shared_gate: bool = True):
+                 table_vocab: int = 0, shared_gate: bool = True, corrected: bool = True):
         """gated False: an expert is W_down max(W_up h, 0)^2 (checkpoint names e<i>.up / e<i>.down). sigmoid: scores are each
         entry's own sigmoid instead of a softmax over the entries. renorm False: the chosen scores are the weights as they are.
         table_vocab > 0: there is no router; row `token id` of `table` [table_vocab, top] (integers) names the token's experts,
-        each with the weight 1 / top, and forward() takes the token ids. shared_gate False: the shared expert is added as it is."""
+        each with the weight 1 / top, and forward() takes the token ids. shared_gate False: the shared expert is added as it is.
+        corrected False: choices go by the scores themselves (no `correction` tensor)."""
         super().__init__()
         self.table_vocab, self.shared_gate = int(table_vocab), bool(shared_gate) and not table_vocab
         self.gated, self.sigmoid, self.renorm = bool(gated), bool(sigmoid), bool(renorm)
@@ -604,7 +757,7 @@ class RoutedExperts(nn.Module):
             self.table = _param(table_vocab, top, dtype=torch.int32)
         else:
             self.router = _param(total + (1 if shared_ff and self.shared_gate else 0), width, dtype=torch.float32)
-            self.correction = _param(total, dtype=torch.float32)
+            self.correction = _param(total, dtype=torch.float32) if corrected else None
         self.w_gu, self.w_down = _param(experts, (2 if gated else 1) * ff, width), _param(experts, width, ff)
         if shared_ff:
             self.s_gu, self.s_down = _param(2 * shared_ff, width), _param(width, shared_ff)
@@ -612,7 +765,9 @@ class RoutedExperts(nn.Module):
     def named_loaders(self) -> dict:
         total, ff = self.E + self.ident, self.ff
         out = {"table": _copy_into(self.table)} if self.table_vocab else \
-            {"router": _copy_into(self.router[:total]), "correction": _copy_into(self.correction)}
+            {"router": _copy_into(self.router[:total])}
+        if not self.table_vocab and self.correction is not None:
+            out["correction"] = _copy_into(self.correction)
         for e in range(self.E):
             if self.gated:
                 out[f"e{e}.gate"] = _copy_into(self.w_gu[e, :ff])
@@ -628,7 +783,8 @@ class RoutedExperts(nn.Module):
                 out["shared.sg"] = _copy_into(self.router[total:])
         return out
 
-    def forward(self, xh: torch.Tensor, tokens: torch.Tensor | None = None) -> torch.Tensor:
+    def forward(self, xh: torch.Tensor, tokens: torch.Tensor | None = None, res: torch.Tensor | None = None) -> torch.Tensor:
+        """The mixture's output; with `res` (the 32-bit residual) it is added there and the new residual is returned instead."""
         n, width = xh.shape
         total = self.E + self.ident
         if self.table_vocab:
@@ -648,8 +804,11 @@ class RoutedExperts(nn.Module):
             sact = torch.empty(n, self.shared_ff, dtype=xh.dtype, device=xh.device)
             ops_seq.glu_act(F.linear(xh, self.s_gu), self.shared_ff, sact, kind=0)
             shared, gate = F.linear(sact, self.s_down), (z[:, total:] if self.shared_gate else None)
+        if res is not None and xh.dtype == torch.float32:
+            ops_seq.moe_combine(rows, plan, wts, xh, shared, gate, None, res)
+            return res
         out = torch.empty(n, width, dtype=xh.dtype, device=xh.device)
-        ops_seq.moe_combine(rows, plan, wts, xh, shared, gate, out)
+        ops_seq.moe_combine(rows, plan, wts, xh, shared, gate, out, res)
         return out
 
 

@@ -15,7 +15,7 @@ import torch
 
 from . import build as _build
 
-ABI_VERSION = 5
+ABI_VERSION = 6
 _P, _I, _L, _F = c_void_p, c_int, c_int64, c_float
 
 SIGNATURES = {
@@ -36,11 +36,19 @@ SIGNATURES = {
     "nvs_ssd_scan_workspace": (c_int64, [_I, _I, _I, _I, _L]),
     "nvs_ssd_scan": (c_int, [_P, _P, _L, _L, _I, _P, _P, _P, _I, _I, _I, _I, _P, _P, _P, _I, _L, _L, _P, _P, _P, _L, _P]),
     "nvs_decay_scan": (c_int, [_P, _L, _L, _L, _L, _I, _P, _I, _I, _I, _P, _P, _P, _I, _L, _L, _P, _P, _P, _L, _P]),
-    "nvs_gated_group_norm": (c_int, [_P, _P, _L, _I, _P, _I, _I, _F, _I, _L, _P, _P, _P]),
+    "nvs_gated_group_norm": (c_int, [_P, _P, _L, _I, _P, _I, _I, _I, _F, _I, _L, _P, _P, _P]),
+    "nvs_delta_scan": (c_int, [_P, _L, _P, _L, _L, _L, _P, _L, _I, _P, _P, _F, _I, _I, _I, _I, _I, _P, _P, _P, _I, _L, _L, _P, _P, _P]),
+    "nvs_delta_force": (None, [_I]),
+    "nvs_embed_norm": (c_int, [_P, _I, _P, _L, _I, _P, _F, _P, _P]),
+    "nvs_shift_norm": (c_int, [_P, _P, _P, _P, _P, _I, _P, _P, _P, _P, _I, _L, _I, _F, _P, _P, _P, _P]),
+    "nvs_gated_lookup": (c_int, [_P, _L, _P, _L, _L, _I, _P, _I, _L, _P, _P]),
+    "nvs_qk_rows": (c_int, [_P, _L, _I, _P, _P, _L, _I, _P, _F, _I, _I, _I, _I, _P, _P, _P, _I, _L, _P, _P, _P, _I, _I, _P, _L, _P, _P, _P, _P]),
+    "nvs_pool_rows": (c_int64, [_I, _I]),
+    "nvs_pool_blocks": (c_int, [_P, _P, _I, _I, _I, _I, _I, _I, _P, _P, _P, _L, _P, _L, _P, _P, _P]),
     "nvs_knorm_kvstore": (c_int, [_P, _P, _L, _I, _P, _F, _I, _I, _I, _I, _P, _P, _P, _I, _L, _P, _P, _P]),
     "nvs_window_attn_force_scalar": (None, [_I]),
-    "nvs_window_attn": (c_int, [_P, _L, _P, _F, _P, _L, _I, _I, _P, _P, _P, _L, _I, _P, _P, _P, _I, _L, _I, _I, _I, _I, _F, _I,
-                                _I, _P, _I, _P, _F, _I, _P, _P]),
+    "nvs_window_attn": (c_int, [_P, _L, _P, _F, _P, _P, _L, _I, _I, _P, _P, _P, _L, _I, _P, _P, _P, _I, _L, _I, _I, _I, _I, _F, _F, _I,
+                                _I, _I, _P, _P, _P, _I, _P, _F, _I, _P, _P]),
     "nvs_add_group_norm": (c_int, [_P, _P, _F, _P, _P, _L, _P, _I, _I, _I, _F, _I, _P, _P]),
     "nvs_scale_softcap": (c_int, [_P, _I, _F, _F, _L, _P, _P]),
     "nvs_latent_prep": (c_int, [_P, _L, _I, _I, _I, _P, _P, _I, _I, _I, _P, _P, _P, _I, _I, _F, _F, _I, _P, _P, _P, _L, _P]),
@@ -51,7 +59,7 @@ SIGNATURES = {
     "nvs_moe_plan": (c_int, [_P, _L, _I, _I, _I, _P, _P, _P, _P]),
     "nvs_moe_gemm": (c_int, [_P, _L, _P, _I, _I, _I, _I, _P, _P, _L, _I, _P, _L, _P]),
     "nvs_moe_force_plain": (None, [_I]),
-    "nvs_moe_combine": (c_int, [_P, _L, _P, _P, _I, _P, _L, _P, _P, _L, _I, _L, _I, _P, _P]),
+    "nvs_moe_combine": (c_int, [_P, _L, _P, _P, _I, _P, _L, _P, _P, _L, _I, _L, _I, _P, _P, _P]),
 }
 
 _lib = None
@@ -213,15 +221,17 @@ def ssd_scan(xbc: torch.Tensor, proj: torch.Tensor, dt_col: int, dt_bias, A_log,
 
 
 def gated_group_norm(y: torch.Tensor, z: torch.Tensor, w: torch.Tensor, groups: int, eps: float, out: torch.Tensor,
-                     norm_first: bool = False, den: torch.Tensor | None = None):
-    """out = group_rms(y * silu(z)) * w, or with norm_first group_rms(y) * w * sigmoid(z); den [n, groups] (32-bit, norm_first only):
-    group g of row t is divided by den[t, g] before anything else."""
+                     norm_first: bool = False, den: torch.Tensor | None = None, silu: bool = False):
+    """out = group_rms(y * silu(z)) * w, or with norm_first group_rms(y) * w * sigmoid(z) (silu: * silu(z)); den [n, groups] (32-bit,
+    norm_first only): group g of row t is divided by den[t, g] before anything else. w has an entry per column, or, shared by the
+    groups, per column of a group."""
     lib = load_library()
     n, inner = y.shape
     assert y.dtype == torch.float32 and y.is_contiguous() and z.shape == (n, inner) and z.stride(1) == 1
-    assert w.numel() == inner and out.shape == (n, inner) and out.is_contiguous()
+    assert w.numel() in (inner, inner // groups) and out.shape == (n, inner) and out.is_contiguous() and (norm_first or not silu)
     assert den is None or (norm_first and den.dtype == torch.float32 and den.shape == (n, groups) and den.is_contiguous())
-    _check(lib.nvs_gated_group_norm(_ptr(y), _ptr(z), z.stride(0), _same(z, w, out), _ptr(w), inner, groups, eps, int(norm_first), n,
+    _check(lib.nvs_gated_group_norm(_ptr(y), _ptr(z), z.stride(0), _same(z, w, out), _ptr(w), w.numel(), inner, groups, eps,
+                                    2 if silu else int(norm_first), n,
                                     _ptr(den), _ptr(out), _stream()))
 
 
@@ -253,12 +263,18 @@ def knorm_kvstore(k: torch.Tensor, v: torch.Tensor, knorm: torch.Tensor | None, 
 def window_attn(q: torch.Tensor, qnorm: torch.Tensor | None, eps: float, gate: torch.Tensor | None, k_cache, v_cache,
                 block_tables: torch.Tensor, block_size: int, por: Portions, H: int, G: int, d: int, dv: int, scale: float,
                 window: int, out: torch.Tensor, chunk: int = 0, rot_freq: torch.Tensor | None = None, gate_per_head: bool = False,
-                sink: torch.Tensor | None = None, q_temp: tuple[float, int] | None = None):
+                sink: torch.Tensor | None = None, q_temp: tuple[float, int] | None = None, q_row: torch.Tensor | None = None,
+                softcap: float = 0.0, pool: int = 0, pool_k: torch.Tensor | None = None, pool_v: torch.Tensor | None = None):
     """window > 0: the last `window` positions; chunk > 0: the query's own block of `chunk` positions; neither: causal.
     rot_freq [r / 2] (32-bit): the first r entries of every query head turn in interleaved pairs by position * rot_freq.
     gate [n, H * dv], or [n, H] with gate_per_head: out *= sigmoid(gate). sink [H] (32-bit): head h's softmax denominator also holds
-    exp(sink[h]). q_temp (coef, every): the query at position p is multiplied by 1 + coef * ln(floor((p + 1) / every) + 1)."""
+    exp(sink[h]). q_temp (coef, every): the query at position p is multiplied by 1 + coef * ln(floor((p + 1) / every) + 1).
+    q_row [n] (32-bit, from qk_rows): qnorm [H * d] belongs to the whole projection and row t's factor is q_row[t]. softcap > 0:
+    scores become softcap * tanh(score / softcap). pool > 0: a query also sees the mean key and value (pool_blocks) of every
+    block of `pool` positions that lies wholly before its window."""
     lib = load_library()
+    assert q_row is None or (q_row.dtype == torch.float32 and q_row.numel() == por.n and qnorm is not None and qnorm.numel() == H * d)
+    assert not pool or (pool_k.is_contiguous() and pool_v.is_contiguous() and window > 0)
     n = por.n
     assert q.shape == (n, H * d) and q.stride(1) == 1 and out.shape == (n, H * dv) and out.is_contiguous()
     assert gate is None or (gate.shape == (n, H if gate_per_head else H * dv) and gate.stride(1) == 1)
@@ -266,23 +282,115 @@ def window_attn(q: torch.Tensor, qnorm: torch.Tensor | None, eps: float, gate: t
     assert tuple(k_cache.shape[1:]) == (G, d) and tuple(v_cache.shape[1:]) == (G, dv)
     assert sink is None or (sink.dtype == torch.float32 and sink.numel() == H and sink.is_contiguous() and sink.is_cuda)
     qt_coef, qt_every = (float(q_temp[0]), int(q_temp[1])) if q_temp else (0.0, 0)
-    _check(lib.nvs_window_attn(_ptr(q), q.stride(0), _ptr(qnorm), eps, _ptr(gate), gate.stride(0) if gate is not None else 0,
+    _check(lib.nvs_window_attn(_ptr(q), q.stride(0), _ptr(qnorm), eps, _ptr(q_row), _ptr(gate), gate.stride(0) if gate is not None else 0,
                                int(gate_per_head), _same(q, qnorm, gate, k_cache, v_cache, out), _ptr(k_cache), _ptr(v_cache), _ptr(block_tables),
                                block_tables.stride(0), block_size, _ptr(por.cu_q), _ptr(por.ctx0), _ptr(por.tseq), por.nseq, n, H,
-                               G, d, dv, scale, window, chunk, _ptr(rot_freq), _rotation(rot_freq), _ptr(sink), qt_coef, qt_every, _ptr(out),
+                               G, d, dv, scale, softcap, window, chunk, pool, _ptr(pool_k), _ptr(pool_v), _ptr(rot_freq), _rotation(rot_freq),
+                               _ptr(sink), qt_coef, qt_every, _ptr(out), _stream()))
+
+
+def qk_rows(q: torch.Tensor, k: torch.Tensor | None, v: torch.Tensor | None, knorm: torch.Tensor | None, eps: float, G: int, d: int, dv: int,
+            block_size: int, slots: torch.Tensor, k_cache, v_cache, pos: torch.Tensor, rot_freq: torch.Tensor | None, por: Portions,
+            block_tables: torch.Tensor, pool: int = 0, pool_k: torch.Tensor | None = None, pool_v: torch.Tensor | None = None) -> torch.Tensor:
+    """Norm over whole projections: returns the factors [n] of the query rows; with k / v (column ranges of one projection) the key
+    rows are normed, rotated and stored with the values, and with `pool` the blocks that end in this step are averaged."""
+    lib = load_library()
+    n = q.shape[0]
+    q_row = torch.empty(n, dtype=torch.float32, device=q.device)
+    assert q.stride(1) == 1 and pos.dtype == torch.int64 and pos.numel() >= n and pos.is_contiguous() and slots.dtype == torch.int32
+    single = por.n == por.nseq                        # one token per portion: the store's workgroups finish the blocks themselves
+    if k is not None:
+        assert k.shape == (n, G * d) and v.shape == (n, G * dv) and k.stride(1) == 1 and v.stride(1) == 1 and k.stride(0) == v.stride(0)
+        assert knorm.numel() == G * d and k_cache.is_contiguous() and v_cache.is_contiguous() and k_cache.shape[0] % block_size == 0
+        assert tuple(k_cache.shape[1:]) == (G, d) and tuple(v_cache.shape[1:]) == (G, dv)
+    _check(lib.nvs_qk_rows(_ptr(q), q.stride(0), q.shape[1], _ptr(k), _ptr(v), k.stride(0) if k is not None else 0, _same(q, k, v, knorm),
+                           _ptr(knorm), eps, G, d, dv, block_size, _ptr(slots), _ptr(pos), _ptr(rot_freq), _rotation(rot_freq), n, _ptr(q_row),
+                           _ptr(k_cache), _ptr(v_cache), pool, int(single), _ptr(block_tables), block_tables.stride(0), _ptr(por.tseq),
+                           _ptr(pool_k), _ptr(pool_v), _stream()))
+    if k is not None and pool and not single:
+        pool_blocks(k_cache, v_cache, G, d, dv, block_size, pool, slots, pos, block_tables, por, pool_k, pool_v)
+    return q_row
+
+
+def pool_rows(block_size: int, pool: int) -> int:
+    """Blocks of `pool` tokens that a page of block_size tokens has room for (whole units of 8)."""
+    return -(-block_size // (8 * pool)) * 8
+
+
+def pool_blocks(k_cache, v_cache, G: int, d: int, dv: int, block_size: int, pool: int, slots: torch.Tensor, pos: torch.Tensor,
+                block_tables: torch.Tensor, por: Portions, pool_k: torch.Tensor, pool_v: torch.Tensor):
+    """Means of the cached keys / values over the blocks of `pool` positions that end in this step."""
+    lib = load_library()
+    rows = pool_rows(block_size, pool) * (k_cache.shape[0] // block_size)
+    assert pool_k.is_contiguous() and pool_k.numel() == rows * G * d and pool_v.is_contiguous() and pool_v.numel() == rows * G * dv
+    assert pos.dtype == torch.int64 and slots.dtype == torch.int32 and block_tables.dtype == torch.int32
+    _check(lib.nvs_pool_blocks(_ptr(k_cache), _ptr(v_cache), _same(k_cache, v_cache, pool_k, pool_v), G, d, dv, block_size, pool, _ptr(slots),
+                               _ptr(pos), _ptr(block_tables), block_tables.stride(0), _ptr(por.tseq), por.n, _ptr(pool_k), _ptr(pool_v),
                                _stream()))
+
+
+def embed_norm(table: torch.Tensor, ids: torch.Tensor, w: torch.Tensor, eps: float, x: torch.Tensor):
+    """x (32-bit) = rms(table[ids]) * w."""
+    lib = load_library()
+    n, width = ids.numel(), table.shape[1]
+    assert x.dtype == torch.float32 and x.shape == (n, width) and x.is_contiguous() and table.is_contiguous() and ids.dtype == torch.int64
+    _check(lib.nvs_embed_norm(_ptr(table), _same(table, w), _ptr(ids), n, width, _ptr(w), eps, _ptr(x), _stream()))
+
+
+def shift_norm(x: torch.Tensor, a: torch.Tensor | None, wa: torch.Tensor | None, w: torch.Tensor, mu: torch.Tensor, eps: float, por: Portions,
+               state: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+    """y = x + a (wa None) or x + rms(a) * wa; h = rms(y) * w; out = h + (h of the previous token - h) * mu, with the last h of every
+    sequence kept in state [nslots, width]. Returns y (x itself when there is nothing to add)."""
+    lib = load_library()
+    n, width = x.shape
+    assert n == por.n and x.dtype == torch.float32 and x.is_contiguous() and out.shape == x.shape and out.is_contiguous()
+    assert a is None or (a.shape == x.shape and a.is_contiguous())
+    assert w.numel() == width and mu.numel() == width and (wa is None or wa.numel() == width)
+    assert state.dtype == torch.float32 and state.is_contiguous() and tuple(state.shape[1:]) == (width,)
+    y = torch.empty_like(x) if a is not None else x
+    _check(lib.nvs_shift_norm(_ptr(x), _ptr(a), _ptr(wa), _ptr(w), _ptr(mu), _same(out, a, wa, w, mu), _ptr(por.cu_q), _ptr(por.ctx0),
+                              _ptr(por.slot), _ptr(por.tseq), por.nseq, n, width, eps, _ptr(state), _ptr(y), _ptr(out), _stream()))
+    return y
+
+
+def gated_lookup(z: torch.Tensor, table: torch.Tensor, col0: int, ids: torch.Tensor) -> torch.Tensor:
+    """gelu_tanh(z) * table[ids, col0 : col0 + dim], z [n, dim]."""
+    lib = load_library()
+    n, dim = z.shape
+    assert z.stride(1) == 1 and table.is_contiguous() and ids.dtype == torch.int64 and ids.numel() == n
+    out = torch.empty(n, dim, dtype=z.dtype, device=z.device)
+    _check(lib.nvs_gated_lookup(_ptr(z), z.stride(0), _ptr(table), table.shape[1], col0, _same(z, table), _ptr(ids), dim, n, _ptr(out), _stream()))
+    return out
+
+
+def delta_scan(qkv: torch.Tensor, gates: torch.Tensor, b_col: int, a_col: int, decays: torch.Tensor | None, A_log: torch.Tensor,
+               dt_bias: torch.Tensor, q_scale: float, heads: int, G: int, dk: int, dv: int, por: Portions, S: torch.Tensor, y: torch.Tensor):
+    """The gated delta rule (see include/nvl_seq.h) on qkv [n, 2 G dk + heads dv]; beta from columns b_col of `gates`; one decay per head
+    from columns a_col of `gates` (decays None), or per head and key channel from columns a_col of `decays`. S [nslots, heads, dv, dk]."""
+    lib = load_library()
+    n = por.n
+    assert qkv.shape == (n, 2 * G * dk + heads * dv) and qkv.stride(1) == 1 and gates.shape[0] == n and gates.stride(1) == 1
+    assert decays is None or (decays.shape[0] == n and decays.stride(1) == 1)
+    assert A_log.dtype == torch.float32 and A_log.numel() == heads and dt_bias.dtype == torch.float32
+    assert dt_bias.numel() == (heads if decays is None else heads * dk) and dt_bias.is_contiguous()
+    assert S.dtype == torch.float32 and S.is_contiguous() and tuple(S.shape[1:]) == (heads, dv, dk)
+    assert y.dtype == torch.float32 and y.is_contiguous() and y.shape == (n, heads * dv)
+    _check(lib.nvs_delta_scan(_ptr(qkv), qkv.stride(0), _ptr(gates), gates.stride(0), b_col, a_col, _ptr(decays),
+                              decays.stride(0) if decays is not None else 0, _same(qkv, gates, decays), _ptr(A_log), _ptr(dt_bias), q_scale,
+                              int(decays is not None), heads, G, dk, dv, _ptr(por.cu_q), _ptr(por.ctx0), _ptr(por.slot), por.nseq, n, por.max_q,
+                              _ptr(S), _ptr(y), _stream()))
 
 
 def add_group_norm(x: torch.Tensor, w: torch.Tensor | None, groups: int, eps: float, out: torch.Tensor | None,
                    a: torch.Tensor | None = None, b: torch.Tensor | None = None, a_mult: float = 1.0, center: bool = False):
     """x += a_mult * a + b (in place; a in the activation type, b 32-bit, both optional), then out = group_rms(x) * w (out None:
-    adds only); center: every group's mean is taken off first (layer norm without bias)."""
+    adds only; w None: out is the sum itself in the activation type); center: every group's mean is taken off first (layer norm without bias)."""
     lib = load_library()
     n, width = x.shape
     assert x.dtype == torch.float32 and x.is_contiguous()
     assert a is None or (a.shape == x.shape and a.is_contiguous())
     assert b is None or (b.shape == x.shape and b.is_contiguous() and b.dtype == torch.float32)
-    assert out is None or (out.shape == x.shape and out.is_contiguous() and w is not None and w.numel() == width)
+    assert out is None or (out.shape == x.shape and out.is_contiguous() and (w is None or w.numel() == width))
     ref = out if out is not None else a
     assert ref is not None, "nothing to do"
     _check(lib.nvs_add_group_norm(_ptr(x), _ptr(a), a_mult, _ptr(b), None, n, _ptr(w) if out is not None else None, _same(ref, a, w, out),
@@ -479,15 +587,18 @@ def moe_gemm(x: torch.Tensor, w: torch.Tensor, plan: MoePlan, glu: bool, out: to
 
 
 def moe_combine(rows: torch.Tensor, plan: MoePlan, wts: torch.Tensor, h: torch.Tensor, shared: torch.Tensor | None,
-                shared_gate: torch.Tensor | None, out: torch.Tensor):
-    """out[t] = sum_k wts[t, k] * (row of the pair, or h[t] for a pass-through choice) + sigmoid(shared_gate[t]) * shared[t]."""
+                shared_gate: torch.Tensor | None, out: torch.Tensor | None, res: torch.Tensor | None = None):
+    """out[t] = sum_k wts[t, k] * (row of the pair, or h[t] for a pass-through choice) + sigmoid(shared_gate[t]) * shared[t]. With res
+    [n, width] (32-bit): res += that sum, and out (may be None) is the new res in the activation type."""
     lib = load_library()
     n, width = h.shape
     top = wts.shape[1]
-    assert rows.stride(1) == 1 and rows.shape[1] == width and h.stride(1) == 1 and out.shape == (n, width) and out.is_contiguous()
+    assert rows.stride(1) == 1 and rows.shape[1] == width and h.stride(1) == 1
+    assert (out is None and res is not None) or (out.shape == (n, width) and out.is_contiguous())
+    assert res is None or (res.dtype == torch.float32 and res.shape == (n, width) and res.is_contiguous())
     assert wts.dtype == torch.float32 and wts.is_contiguous() and plan.pair_row.shape == (n, top)
     assert shared is None or (shared.shape == (n, width) and shared.is_contiguous())
     assert shared_gate is None or (shared is not None and shared_gate.dtype == torch.float32 and shared_gate.shape[0] == n)
     _check(lib.nvs_moe_combine(_ptr(rows), rows.stride(0), _ptr(plan.pair_row), _ptr(wts), top, _ptr(h), h.stride(0), _ptr(shared),
                                _ptr(shared_gate), shared_gate.stride(0) if shared_gate is not None else 0, _same(rows, h, shared, out), n,
-                               width, _ptr(out), _stream()))
+                               width, _ptr(res), _ptr(out), _stream()))

@@ -78,6 +78,17 @@ def _lobidra_build(config, dtype=None):
     return LobidraForCausalLM(config, dtype)
 
 
+def _ligidra_config(path: str, raw: dict):
+    from .ligidra import LigidraConfig
+    from .weights import checkpoint_shapes
+    return LigidraConfig(raw, checkpoint_shapes(path))
+
+
+def _ligidra_build(config, dtype=None):
+    from .ligidra import LigidraForCausalLM
+    return LigidraForCausalLM(config, dtype)
+
+
 REGISTRY: dict[str, ModelSpec] = {
     "Qwen3ForCausalLM": ModelSpec("Qwen3ForCausalLM", _qwen3_config, _qwen3_build),
     "Qwen2ForCausalLM": ModelSpec("Qwen2ForCausalLM", _qwen3_config, _qwen3_build),      # same module tree, biased qkv, no q/k norm
@@ -88,6 +99,8 @@ REGISTRY: dict[str, ModelSpec] = {
     "Pefazen": ModelSpec("Pefazen", _pefazen_config, _pefazen_build, stateful=True, block_multiple=16,
                          dtypes=("bfloat16", "float32")),
     "Lobidra": ModelSpec("Lobidra", _lobidra_config, _lobidra_build, stateful=True, block_multiple=16,
+                         dtypes=("bfloat16", "float32")),
+    "Ligidra": ModelSpec("Ligidra", _ligidra_config, _ligidra_build, stateful=True, block_multiple=16,
                          dtypes=("bfloat16", "float32")),
 }
 

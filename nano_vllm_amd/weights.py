@@ -145,6 +145,17 @@ def _assign(param: nn.Parameter, tensor: torch.Tensor, shard) -> None:
         loader(param, tensor, shard)
 
 
+def checkpoint_shapes(path: str) -> dict[str, tuple]:
+    """Tensor names -> shapes of every *.safetensors under `path`, from the files' headers (empty when there are none): for sizes that
+    a family's configuration leaves to its tensors."""
+    from safetensors import safe_open
+    out = {}
+    for file in sorted(glob(os.path.join(path, "*.safetensors"))):
+        with safe_open(file, "pt", "cpu") as f:
+            out.update({name: tuple(f.get_slice(name).get_shape()) for name in f.keys()})
+    return out
+
+
 def load_model(model: nn.Module, path: str) -> int:
     """Load every tensor of every *.safetensors under `path`. Returns the number loaded."""
     from safetensors import safe_open
