@@ -1,7 +1,6 @@
 // The gated delta rule (see nvs_delta_scan in include/nvl_seq.h): a matrix state per head whose write is the ERROR of what the
 // state already answers for the key. Everything from the unit norms on is 32-bit.
 #include "seq_common.h"
-#include <stdlib.h>
 
 namespace {
 
@@ -184,6 +183,356 @@ void launch_walk(const DeltaArgs& A, int nseq, hipStream_t stream) {
   }
 }
 
+// ---- in chunks of 16 tokens -------------------------------------------------------------------------------------------
+// With G_t the product of a chunk's decays up to token t (inclusive) and S the state before the chunk, the chunk's writes u_t solve a
+// unit lower triangular system, and outputs and the next state are plain products:
+//   u_t + beta_t sum_{j<t} A_tj u_j = beta_t (v_t - (G_t k_t) . S),   A_tj = sum_c k_tc k_jc (G_t / G_j)_c
+//   o_t = (G_t q_t) . S + sum_{j<=t} M_tj u_j,                         M_tj = sum_c q_tc k_jc (G_t / G_j)_c
+//   S  <- G_C S + sum_j (G_C / G_j k_j) u_j^T
+// All products run on v_mfma_f32_16x16x4_f32. A workgroup serves one (portion, head) and up to 8 x 16 value columns: four wavefronts
+// prepare chunk n + 1 (unit vectors, decays, A, M, the inverse T of the system) while the others, 16 columns each with their dk x 16
+// piece of the state in accumulators, work on chunk n. The state piece is a B operand as it stands — an accumulator register r holds
+// rows 4 (lane / 16) + r of its tile, so contraction step r of a tile takes A's column 4 (lane / 16) + r — and so are u and the
+// output, so nothing is ever exchanged between lanes. Four phases per chunk, a workgroup barrier after each:
+//   columns:  O = Q S | U = T (V - P), O += M U, store | S = G_C S + K^T U | P = K S of the next chunk
+//   prepare:  unit vectors, decays | decay products, G k, G q | A, M | T; K^T, G_C
+// Decay products are multiplied up (no exponential of a difference). Per-channel decays: A and M are products of G k with k / G as
+// long as no channel decays by more than 1e-20 within the chunk; otherwise every pair (j, t) is walked with the product G_t / G_j
+// carried along. A partial chunk is filled with tokens that change nothing (k = q = v = 0, beta = 0, decay 1).
+typedef __attribute__((ext_vector_type(4))) float f32x4_t;
+constexpr int CHUNK = 16, PREP = 256, MST = 20;      // MST: row stride of the 16 x 16 matrices in LDS (float4-aligned)
+
+__device__ __forceinline__ f32x4_t mfma4(float a, float b, f32x4_t c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
+
+template <int DKT, bool CH>
+struct ChunkLds {
+  static constexpr int DKP = 16 * DKT, LD = DKP + 4;
+  float kg[CHUNK][LD], qg[CHUNK][LD];               // G k, G q
+  float kn[CHUNK][LD], qn[CHUNK][LD];               // unit vectors
+  float g[CH ? CHUNK : 1][LD];                      // decays per channel, or [0][t] per token
+  float ki[CH ? CHUNK : 1][LD];                     // k / G
+  float kt[DKP][MST];                               // (G_C / G_j k_j) transposed: channel, token
+  float gc[DKP];                                    // G_C
+  float part[4][CHUNK][MST];                        // A (0, 1) and M (2, 3) in two halves of the channels each
+  float ratio[CH ? 1 : CHUNK][MST];                 // G_t / G_j of per-head decays
+  float T[CHUNK][MST], M[CHUNK][MST], L[CHUNK][MST];
+  float beta[CHUNK];
+  int strong;                                       // chunk number + 1 of the last chunk with a channel below the limit
+};
+
+template <typename T, int DKT, bool CH>
+__global__ __launch_bounds__(768) void delta_chunk_kernel(const DeltaArgs A) {
+  typedef ChunkLds<DKT, CH> Lds;
+  constexpr int DKP = Lds::DKP;
+  extern __shared__ __attribute__((aligned(16))) char chunk_lds[];
+  Lds& W = *(Lds*)chunk_lds;
+  const int s = blockIdx.y, h = blockIdx.x, tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int64_t q0 = A.cu_q[s], q1 = A.cu_q[s + 1];
+  if (q1 <= q0) return;
+  const int dk = A.dk, dv = A.dv, grp = h / (A.heads / A.G);
+  const int li = lane & 15, lq = lane >> 4;
+  const bool prep = wave < 4;
+  const int nch = (int)((q1 - q0 + CHUNK - 1) / CHUNK);
+  if (tid == 0) W.strong = 0;
+
+  // ---- prepare: thread (token pt, lane pl of 16) holds channels pl + 16 e of its token
+  const int pt = (tid >> 4) & 15, pl = tid & 15;
+  const T* qp = (const T*)A.qkv + (int64_t)grp * dk;
+  const T* kp = (const T*)A.qkv + (int64_t)(A.G + grp) * dk;
+  const T* ap = CH ? (const T*)A.decays + A.a_col + (int64_t)h * dk : (const T*)A.gates + A.a_col + h;
+  const T* bp = (const T*)A.gates + A.b_col + h;
+  const float* dtb = A.dt_bias + (CH ? (int64_t)h * dk : h);
+  const float rate = -expf(A.A_log[h]);
+  float rk_[DKT], rq_[DKT], ra_[CH ? DKT : 1], rb = 0.f;
+  auto load = [&](int n) {
+    const int64_t t = q0 + (int64_t)n * CHUNK + pt;
+    const bool in = t < q1;
+#pragma unroll
+    for (int e = 0; e < DKT; ++e) {
+      const int c = pl + 16 * e;
+      const bool ok = in && c < dk;
+      rk_[e] = ok ? ldf(kp + t * A.qkv_stride + c) : 0.f;
+      rq_[e] = ok ? ldf(qp + t * A.qkv_stride + c) : 0.f;
+      if (CH) ra_[e] = ok ? ldf(ap + t * A.decays_stride + c) : 0.f;
+    }
+    if (!CH) ra_[0] = in ? ldf(ap + t * A.gates_stride) : 0.f;
+    rb = in ? ldf(bp + t * A.gates_stride) : 0.f;
+  };
+  auto stage = [&](int n) {
+    const bool in = q0 + (int64_t)n * CHUNK + pt < q1;
+    float sk = 0.f, sq = 0.f;
+#pragma unroll
+    for (int e = 0; e < DKT; ++e) sk += rk_[e] * rk_[e], sq += rq_[e] * rq_[e];
+#pragma unroll
+    for (int o = 8; o > 0; o >>= 1) sk += __shfl_xor(sk, o, 64), sq += __shfl_xor(sq, o, 64);
+    const float fk = 1.f / sqrtf(sk + UNIT_EPS), fq = A.q_scale / sqrtf(sq + UNIT_EPS);
+#pragma unroll
+    for (int e = 0; e < DKT; ++e) {
+      const int c = pl + 16 * e;
+      W.kn[pt][c] = rk_[e] * fk;
+      W.qn[pt][c] = rq_[e] * fq;
+      if (CH) W.g[pt][c] = in && c < dk ? expf(rate * softplusf_(ra_[e] + dtb[c < dk ? c : 0])) : 1.f;
+    }
+    if (pl == 0) {
+      if (!CH) W.g[0][pt] = in ? expf(rate * softplusf_(ra_[0] + dtb[0])) : 1.f;
+      W.beta[pt] = in ? 1.f / (1.f + expf(-rb)) : 0.f;
+    }
+  };
+  auto products = [&](int n) {                       // G k, G q, k / G: a channel per thread, K and Q parts apart
+    for (int w = tid; w < 2 * DKP; w += PREP) {
+      const int c = w & (DKP - 1);
+      float G = 1.f;
+      if (w < DKP) {
+#pragma unroll
+        for (int t = 0; t < CHUNK; ++t) {
+          G *= CH ? W.g[t][c] : W.g[0][t];
+          const float k = W.kn[t][c];
+          W.kg[t][c] = G * k;
+          if (CH) W.ki[t][c] = k / G;
+        }
+        if (CH && G < 1e-20f) W.strong = n + 1;
+      } else {
+#pragma unroll
+        for (int t = 0; t < CHUNK; ++t) {
+          G *= CH ? W.g[t][c] : W.g[0][t];
+          W.qg[t][c] = G * W.qn[t][c];
+        }
+      }
+    }
+    if (!CH) {
+      float r = 1.f;
+      for (int i = pl + 1; i <= pt; ++i) r *= W.g[0][i];
+      W.ratio[pt][pl] = r;
+    }
+  };
+  auto matrices = [&](int n) {
+    if (CH && W.strong == n + 1) {
+      // pair by pair: thread (token j = pt, lane pl) carries k_j times the decays since j through the later tokens
+      float w[DKT];
+#pragma unroll
+      for (int e = 0; e < DKT; ++e) w[e] = W.kn[pt][pl + 16 * e];
+      for (int t = 0; t < CHUNK; ++t) {
+        float a = 0.f, m = 0.f;
+        if (t >= pt) {
+#pragma unroll
+          for (int e = 0; e < DKT; ++e) {
+            const int c = pl + 16 * e;
+            if (t > pt) w[e] *= W.g[t][c];
+            a += W.kn[t][c] * w[e];
+            m += W.qn[t][c] * w[e];
+          }
+        }
+#pragma unroll
+        for (int o = 8; o > 0; o >>= 1) a += __shfl_xor(a, o, 64), m += __shfl_xor(m, o, 64);
+        if (pl == 0) W.part[0][t][pt] = a, W.part[1][t][pt] = 0.f, W.part[2][t][pt] = m, W.part[3][t][pt] = 0.f;
+      }
+      return;
+    }
+    const int half = wave & 1;
+    const auto& left = wave < 2 ? (CH ? W.kg : W.kn) : (CH ? W.qg : W.qn);
+    const auto& right = *(const float(*)[CHUNK][Lds::LD])(CH ? &W.ki[0][0] : &W.kn[0][0]);
+    f32x4_t acc[2] = {f32x4_t{0.f, 0.f, 0.f, 0.f}, f32x4_t{0.f, 0.f, 0.f, 0.f}};
+#pragma unroll
+    for (int i = 0; i < (DKT + 1) / 2; ++i) {
+      const int tt = half * ((DKT + 1) / 2) + i;
+      if (tt < DKT) {
+        const float4 a = *(const float4*)&left[li][16 * tt + 4 * lq], b = *(const float4*)&right[li][16 * tt + 4 * lq];
+        acc[0] = mfma4(a.x, b.x, acc[0]);
+        acc[1] = mfma4(a.y, b.y, acc[1]);
+        acc[0] = mfma4(a.z, b.z, acc[0]);
+        acc[1] = mfma4(a.w, b.w, acc[1]);
+      }
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) W.part[wave][4 * lq + r][li] = acc[0][r] + acc[1][r];
+  };
+  auto solve = [&]() {
+    if (wave == 0) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {                  // L = beta A below the diagonal
+        const int t = 4 * i + lq;
+        float a = W.part[0][t][li] + W.part[1][t][li];
+        if (!CH) a *= W.ratio[t][li];
+        W.L[t][li] = li < t ? W.beta[t] * a : 0.f;
+      }
+      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "workgroup");
+      __builtin_amdgcn_wave_barrier();
+      float x[CHUNK];                                // column li of (I + L)^-1, row after row
+#pragma unroll
+      for (int t = 0; t < CHUNK; ++t) {
+        float v = t == li ? 1.f : 0.f;
+#pragma unroll
+        for (int j = 0; j < t; ++j) v -= W.L[t][j] * x[j];
+        x[t] = v;
+      }
+      const float b = W.beta[li];
+      if (lq == 0) {
+#pragma unroll
+        for (int t = 0; t < CHUNK; ++t) W.T[t][li] = x[t] * b;
+      }
+    } else if (wave == 1) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int t = 4 * i + lq;
+        float m = W.part[2][t][li] + W.part[3][t][li];
+        if (!CH) m *= W.ratio[t][li];
+        W.M[t][li] = li <= t ? m : 0.f;
+      }
+    } else {
+      for (int c = tid - 128; c < DKP; c += 128) {
+        float D = 1.f, col[CHUNK];
+#pragma unroll
+        for (int t = CHUNK - 1; t >= 0; --t) {
+          col[t] = D * W.kn[t][c];
+          D *= CH ? W.g[t][c] : W.g[0][t];
+        }
+#pragma unroll
+        for (int t = 0; t < CHUNK; t += 4) *(float4*)&W.kt[c][t] = make_float4(col[t], col[t + 1], col[t + 2], col[t + 3]);
+        W.gc[c] = D;
+      }
+    }
+  };
+
+  // the two roles in loops of their own (their registers are then not live together); both meet in the same 1 + 4 (nch + 1) barriers
+  if (prep) {
+    load(0);
+    __syncthreads();
+    for (int n = 0; n <= nch; ++n) {                // chunk n is prepared while chunk n - 1 is worked on
+      const bool next = n < nch;
+      if (next) {
+        stage(n);
+        if (n + 1 < nch) load(n + 1);
+      }
+      __syncthreads();
+      if (next) products(n);
+      __syncthreads();
+      if (next) matrices(n);
+      __syncthreads();
+      if (next) solve();
+      __syncthreads();
+    }
+    return;
+  }
+  // ---- columns: 16 value columns per wavefront
+  const int col = (blockIdx.z * ((blockDim.x >> 6) - 4) + (wave - 4)) * 16 + li;
+  const bool own = col < dv;
+  float* Sc = A.S + (((int64_t)A.slot[s] * A.heads + h) * dv + (own ? col : 0)) * dk;
+  const T* vp = (const T*)A.qkv + (int64_t)2 * A.G * dk + (int64_t)h * dv + col;
+  f32x4_t st[DKT], P = {0.f, 0.f, 0.f, 0.f}, O = {0.f, 0.f, 0.f, 0.f}, U = {0.f, 0.f, 0.f, 0.f};
+  float v[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int i = 0; i < DKT; ++i) st[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+  if (own && A.ctx0[s] != 0) {
+#pragma unroll
+    for (int i = 0; i < DKT; ++i) {
+      const int c = 16 * i + 4 * lq;
+      if ((dk & 3) == 0) {
+        if (c < dk) st[i] = *(const f32x4_t*)(Sc + c);
+      } else {
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (c + r < dk) st[i][r] = Sc[c + r];
+      }
+    }
+  }
+  auto load_v = [&](int n) {
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int64_t t = q0 + (int64_t)n * CHUNK + 4 * lq + r;
+      v[r] = own && t < q1 ? ldf(vp + t * A.qkv_stride) : 0.f;
+    }
+  };
+  auto times_state = [&](const float (&m)[CHUNK][Lds::LD]) {      // m S, [16 tokens x 16 columns]
+    f32x4_t a0 = {0.f, 0.f, 0.f, 0.f}, a1 = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int i = 0; i < DKT; ++i) {
+      const float4 a = *(const float4*)&m[li][16 * i + 4 * lq];
+      a0 = mfma4(a.x, st[i][0], a0);
+      a1 = mfma4(a.y, st[i][1], a1);
+      a0 = mfma4(a.z, st[i][2], a0);
+      a1 = mfma4(a.w, st[i][3], a1);
+    }
+    return a0 + a1;
+  };
+  load_v(0);
+  __syncthreads();
+  for (int n = -1; n < nch; ++n) {
+    const bool next = n + 1 < nch;
+    if (n >= 0) O = times_state(W.qg);
+    __syncthreads();
+    if (n >= 0) {
+      f32x4_t X;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) X[r] = v[r] - P[r];
+      if (next) load_v(n + 1);
+      const float4 t4 = *(const float4*)&W.T[li][4 * lq], m4 = *(const float4*)&W.M[li][4 * lq];
+      U = mfma4(t4.x, X[0], f32x4_t{0.f, 0.f, 0.f, 0.f});
+      U = mfma4(t4.y, X[1], U);
+      U = mfma4(t4.z, X[2], U);
+      U = mfma4(t4.w, X[3], U);
+      O = mfma4(m4.x, U[0], O);
+      O = mfma4(m4.y, U[1], O);
+      O = mfma4(m4.z, U[2], O);
+      O = mfma4(m4.w, U[3], O);
+      if (own) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int64_t t = q0 + (int64_t)n * CHUNK + 4 * lq + r;
+          if (t < q1) A.y[(t * A.heads + h) * dv + col] = O[r];
+        }
+      }
+    }
+    __syncthreads();
+    if (n >= 0) {
+#pragma unroll
+      for (int i = 0; i < DKT; ++i) {
+        const float4 g4 = *(const float4*)&W.gc[16 * i + 4 * lq], a = *(const float4*)&W.kt[16 * i + li][4 * lq];
+        st[i][0] *= g4.x, st[i][1] *= g4.y, st[i][2] *= g4.z, st[i][3] *= g4.w;
+        st[i] = mfma4(a.x, U[0], st[i]);
+        st[i] = mfma4(a.y, U[1], st[i]);
+        st[i] = mfma4(a.z, U[2], st[i]);
+        st[i] = mfma4(a.w, U[3], st[i]);
+      }
+    }
+    __syncthreads();
+    if (next) P = times_state(W.kg);
+    __syncthreads();
+  }
+  if (own) {
+#pragma unroll
+    for (int i = 0; i < DKT; ++i) {
+      const int c = 16 * i + 4 * lq;
+      if ((dk & 3) == 0) {
+        if (c < dk) *(f32x4_t*)(Sc + c) = st[i];
+      } else {
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+          if (c + r < dk) Sc[c + r] = st[i][r];
+      }
+    }
+  }
+}
+
+template <typename T, int DKT, bool CH>
+void launch_chunk_size(const DeltaArgs& A, int nseq, hipStream_t stream) {
+  const int tiles = (A.dv + 15) / 16;
+  // column wavefronts per workgroup: all columns of a head together (they share the preparation) once the (portion, head) pairs
+  // fill the chip, fewer columns per workgroup otherwise
+  int ncw = tiles < 8 ? tiles : 8;
+  while (ncw > 1 && (int64_t)A.heads * nseq * ((tiles + ncw - 1) / ncw) < 384) ncw = (ncw + 1) / 2;
+  const size_t lds = sizeof(ChunkLds<DKT, CH>);
+  if (lds > 48 * 1024) (void)hipFuncSetAttribute((const void*)delta_chunk_kernel<T, DKT, CH>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+  delta_chunk_kernel<T, DKT, CH><<<dim3(A.heads, (unsigned)nseq, (unsigned)((tiles + ncw - 1) / ncw)), dim3(64 * (4 + ncw)), lds, stream>>>(A);
+}
+
+template <typename T, bool CH>
+void launch_chunk(const DeltaArgs& A, int nseq, hipStream_t stream) {
+  if (A.dk <= 32) launch_chunk_size<T, 2, CH>(A, nseq, stream);
+  else if (A.dk <= 64) launch_chunk_size<T, 4, CH>(A, nseq, stream);
+  else if (A.dk <= 128) launch_chunk_size<T, 8, CH>(A, nseq, stream);
+  else launch_chunk_size<T, 16, CH>(A, nseq, stream);
+}
+
 int g_delta_mode = 0;
 
 }  // namespace
@@ -203,7 +552,14 @@ extern "C" int nvs_delta_scan(const void* qkv, int64_t qkv_stride, const void* g
   if (n == 0 || nseq == 0) return NVS_OK;
   DeltaArgs A = {qkv, gates, decays, A_log, dt_bias, cu_q, ctx0, slot, S, y, qkv_stride, gates_stride, b_col, a_col, decays_stride,
                  heads, G, dk, dv, q_scale};
-  if (per_channel) {
+  const bool chunks = dk <= 256 && (g_delta_mode == 2 || (g_delta_mode == 0 && n > nseq && max_q >= CHUNK));
+  if (chunks) {
+    if (per_channel) {
+      NVS_DISPATCH(dtype, launch_chunk<T, true>(A, nseq, (hipStream_t)stream));
+    } else {
+      NVS_DISPATCH(dtype, launch_chunk<T, false>(A, nseq, (hipStream_t)stream));
+    }
+  } else if (per_channel) {
     NVS_DISPATCH(dtype, launch_walk<T, true>(A, nseq, (hipStream_t)stream));
   } else {
     NVS_DISPATCH(dtype, launch_walk<T, false>(A, nseq, (hipStream_t)stream));

@@ -409,3 +409,86 @@ def test_lobidra_checkpoint_names_loaders_and_weights_shared_between_layers():
     assert p.mlp.table_vocab == 29 and not p.mlp.shared_gate and not hasattr(p.mlp, "router") and a.mlp.up.shape == (20, 16)
     # the rotation's table: wavelengths 2 pi and 20 pi against marks at 8 and 16 positions: the first pair stays, the second is slowed
     assert a.mixer.attn.rot_freq.tolist() == [1.0, pytest.approx(0.05)]
+
+
+# ---- Ligidra --------------------------------------------------------------------------------------------------------------
+def lgd_raw():
+    mlp = {"kind": "moe", "expert": {"ff": 10}, "router": {"experts": 3, "top": 2}, "shared": {"ff": 12}}
+    att = {"heads": 4, "kv_heads": 2, "dim": 6, "vdim": 5, "scale": 0.4, "softcap": 9.0, "mask": {"size": 10, "pool": 3},
+           "rot": {"dims": 4, "base": 100.0, "scaling": {"factor": 2.0, "low": 1.0, "high": 2.0, "original": 16}}}
+    dl = {"heads": 4, "kv_heads": 2, "dim": 3, "vdim": 7, "conv": 3}
+    return {"architecture": "Ligidra", "norm": {"eps": 1e-5}, "vocab": 29, "width": 16, "token_side": {"dim": 5},
+            "layers": [{"type": "attention", "mixer": att, "mlp": mlp}, {"type": "delta", "mixer": dl, "mlp": None},
+                       {"type": "channel_delta", "mixer": dict(dl, decay_rank=2, gate_rank=6), "mlp": dict(mlp, shared=None)},
+                       {"type": "attention", "mixer": dict(att, kv_from=0, mask={"size": 7, "pool": 4}), "mlp": mlp}]}
+
+
+def test_ligidra_registry_and_config_checks(tmp_path):
+    from nano_vllm_amd.ligidra import write_synthetic_checkpoint
+    from nano_vllm_amd.registry import REGISTRY, resolve
+    (tmp_path / "config.json").write_text(json.dumps(lgd_raw()))
+    spec, cfg = resolve(str(tmp_path))
+    assert spec is REGISTRY["Ligidra"] and spec.stateful and set(spec.dtypes) == {"bfloat16", "float32"}
+    assert (cfg.vocab_size, cfg.hidden_size, cfg.side_dim, cfg.eps, cfg.ranks(2)) == (29, 16, 5, 1e-5, (2, 6))
+    # with a checkpoint the low ranks are the tensors' own, whatever the configuration says of them
+    write_synthetic_checkpoint(str(tmp_path), lgd_raw())
+    raw = lgd_raw()
+    del raw["layers"][2]["mixer"]["decay_rank"], raw["layers"][2]["mixer"]["gate_rank"]
+    (tmp_path / "config.json").write_text(json.dumps(raw))
+    assert resolve(str(tmp_path))[1].ranks(2) == (2, 6)
+    cases = [(lambda r: r["layers"][0].update(type="lstm"), "mixer type"), (lambda r: r["layers"][0].update(mlp={"kind": "dense"}), "feed-forward kind"),
+             (lambda r: r["layers"][3]["mixer"].update(kv_from=3), "kv_from"), (lambda r: r["layers"][3]["mixer"].update(kv_from=1), "kv_from"),
+             (lambda r: r["layers"].append(dict(r["layers"][3], mixer=dict(r["layers"][3]["mixer"], kv_from=3))), "kv_from")]
+    for change, msg in cases:
+        raw = json.loads(json.dumps(lgd_raw()))
+        change(raw)
+        (tmp_path / "config.json").write_text(json.dumps(raw))
+        with pytest.raises(ValueError, match=msg):
+            resolve(str(tmp_path))
+
+
+def test_ligidra_checkpoint_names_loaders_states_and_summaries():
+    from nano_vllm_amd.ligidra import LigidraConfig, LigidraForCausalLM, random_tensors, tensor_shapes
+    raw = lgd_raw()
+    model = LigidraForCausalLM(LigidraConfig(raw), torch.float32, block_size=16)
+    loaders, shapes = model.named_loaders(), tensor_shapes(raw)
+    assert set(loaders) == set(shapes) and "head" not in shapes
+    assert not any(n in shapes for n in ("l3.mix.k", "l3.mix.v", "l3.mix.k.norm", "l1.norm2", "l2.mlp.shared.up", "l0.mlp.correction", "l0.mlp.shared.sg"))
+    tensors = random_tensors(raw, seed=3)
+    with torch.no_grad():
+        for name, t in tensors.items():
+            assert tuple(t.shape) == tuple(shapes[name])
+            loaders[name](t)
+    assert sum(p.numel() for p in model.parameters()) == sum(int(torch.tensor(s).prod()) for s in shapes.values())
+    own, dl, cd, bor = (layer.mixer for layer in model.layers)
+    # fused in-projections: [q | k | v], [q] for the borrower, [q | k | v | g | a | b], [q | k | v | g1 | a1 | b]
+    assert own.in_w.shape == (24 + 12 + 10, 16) and bor.in_w.shape == (24, 16) and own.in_b is None
+    assert dl.in_w.shape == (6 + 6 + 28 + 28 + 4 + 4, 16) and cd.in_w.shape == (6 + 6 + 28 + 6 + 2 + 4, 16)
+    f = lambda n: tensors[n].float()
+    assert torch.equal(own.in_w[24:36], f("l0.mix.k")) and torch.equal(bor.in_w, f("l3.mix.q")) and torch.equal(own.attn.sink, f("l0.mix.sink"))
+    assert torch.equal(dl.in_w[40:68], f("l1.mix.g")) and torch.equal(dl.in_w[-4:], f("l1.mix.b")) and torch.equal(dl.conv_w[6:12], f("l1.mix.k.conv"))
+    assert torch.equal(cd.in_w[40:46], f("l2.mix.g1")) and torch.equal(cd.in_w[46:48], f("l2.mix.a1")) and torch.equal(cd.a2, f("l2.mix.a2"))
+    assert dl.state_shapes() == {"conv_state": (2, 40), "rec_state": (4, 7, 3)} and model.layers[0].norm1.state_shapes() == {"shift_state": (16,)}
+    # the borrower owns no pages; its blocks have another length than the owner's, so their means are its own
+    assert own.attn.kv_shapes() == ((2, 6), (2, 5)) and bor.attn.kv_shapes() is None and bor.attn.owner is own.attn
+    assert own.attn.page_shapes() == {"pool_k": (8, 2, 6), "pool_v": (1, 2, 5, 8)} and bor.attn.page_shapes() == own.attn.page_shapes()
+    bor.attn.pool = 3
+    assert bor.attn.page_shapes() == {}
+    assert model.layers[2].side.col0 == 10 and model.side_embed.shape == (29, 20)
+
+
+@pytest.mark.parametrize("block,pool", [(16, 1), (16, 3), (16, 16), (64, 5), (64, 12), (64, 100), (48, 7), (256, 16)])
+def test_every_block_of_positions_has_a_place_of_its_own_in_the_pages(block, pool):
+    """Blocks are kept in units of 8, unit u in the page that holds the last token of its first block: when a block is complete the
+    page of its unit exists, and no two units share a place (the arithmetic of the attention kernels, restated)."""
+    from nano_vllm_amd.ops_seq import pool_rows
+    per_page = pool_rows(block, pool) // 8
+    seen = set()
+    for u in range(200):
+        page = (8 * u * pool + pool - 1) // block
+        first = 0 if page * block < pool else (page * block - pool + 8 * pool) // (8 * pool)
+        at = u - first
+        assert 0 <= at < per_page and (page, at) not in seen
+        seen.add((page, at))
+        for b in range(8 * u, 8 * u + 8):
+            assert page <= (b * pool + pool - 1) // block
