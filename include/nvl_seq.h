@@ -51,10 +51,10 @@ int nvs_add_group_norm(float* x, const void* a, float a_mult, const float* b, co
 /* Norms on both sides of a sublayer, on the 32-bit residual. The sublayer's output y[t, :] = a_mult * a[t, :] + a2_mult * a2[t, :]
  * (a2 may be NULL) is divided by its root mean square and multiplied by (w_off + wa), and added: x[t, :] += rms(y) * (w_off + wa);
  * then out[t, :] = rms(x[t, :]) * (w_off + w), the next sublayer's input. a == NULL: nothing is added; out == NULL: the add only.
- * w_off = 1 serves weights that are stored as their distance from one. With rows != NULL nothing is added and out[r, :] is the
- * norm of x[rows[r], :]. a, a2, wa, w, out in `dtype`; every sum in 32-bit. */
+ * w_off = 1 serves weights that are stored as their distance from one. With rows != NULL x is only read: out[r, :] is the norm of
+ * x[rows[r], :], or, with a, of that row with its branch added (the sums go to sum [nrows, width], 32-bit). a, a2, wa, w, out in `dtype`; every sum in 32-bit. */
 int nvs_sandwich_norm(float* x, const void* a, float a_mult, const void* a2, float a2_mult, const void* wa, const int32_t* rows,
-                      int64_t nrows, const void* w, float w_off, int dtype, int width, float eps, void* out, void* stream);
+                      int64_t nrows, const void* w, float w_off, int dtype, int width, float eps, float* sum, void* out, void* stream);
 
 /* x[t, :] = rms(table[ids[t], :]) * w, 32-bit. */
 int nvs_embed_norm(const void* table, int dtype, const int64_t* ids, int64_t n, int width, const void* w, float eps, float* x, void* stream);

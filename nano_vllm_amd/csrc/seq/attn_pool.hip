@@ -7,26 +7,45 @@ namespace {
 
 constexpr int MAX_HEAD_POOL = 1024;
 
-// The mean of the `pool` cached tokens that end at position p into their block's place (see pool_unit); all threads of the
-// workgroup, every kv head. Values are transposed inside a unit of 8 blocks as they are inside a page.
+// The mean of the `pool` cached tokens that end at position p into their block's place (see pool_unit), every kv head: the keys
+// (half 0) or the values (half 1), by all threads of the workgroup. Key rows are read a column per thread; values are transposed
+// inside a page (and inside a unit of 8 blocks), so there LN neighbouring lanes share a column and read its consecutive tokens.
 template <typename T>
-__device__ void pool_block(int p, const int32_t* __restrict__ bt, const T* k_cache, const T* v_cache, int G, int d, int dv,
+__device__ void pool_block(int half, int p, const int32_t* __restrict__ bt, const T* k_cache, const T* v_cache, int G, int d, int dv,
                            int block_size, int pool, T* pool_k, T* pool_v) {
   const int b = p / pool, first = b * pool;
   const int64_t unit = pool_unit(b >> 3, pool, block_size, bt);
   const float inv = 1.f / (float)pool;
   const int nk = G * d, nv = G * dv;
-  for (int c = threadIdx.x; c < nk + nv; c += blockDim.x) {
-    float sum = 0.f;
-    int page = first / block_size, off = first - page * block_size;
-    int64_t pg = bt[page];
-    for (int j = 0; j < pool; ++j) {
-      if (c < nk) sum += ldf(k_cache + (pg * block_size + off) * nk + c);
-      else sum += ldf(v_cache + (pg * nv + (c - nk)) * block_size + off);
-      if (++off == block_size && j + 1 < pool) off = 0, pg = bt[++page];
+  if (half == 0) {
+    for (int c = threadIdx.x; c < nk; c += blockDim.x) {
+      float sum = 0.f;
+      for (int j = first; j <= p;) {                // a run of tokens inside one page at a time
+        const int page = j / block_size, off = j - page * block_size;
+        const int run = block_size - off < p + 1 - j ? block_size - off : p + 1 - j;
+        const T* src = k_cache + ((int64_t)bt[page] * block_size + off) * nk + c;
+#pragma unroll 8
+        for (int i = 0; i < run; ++i) sum += ldf(src + (int64_t)i * nk);
+        j += run;
+      }
+      stf(pool_k + (unit * 8 + (b & 7)) * nk + c, sum * inv);
     }
-    if (c < nk) stf(pool_k + (unit * 8 + (b & 7)) * nk + c, sum * inv);
-    else stf(pool_v + (unit * nv + (c - nk)) * 8 + (b & 7), sum * inv);
+    return;
+  }
+  int ln = 1;
+  while (ln < pool && ln < 16) ln <<= 1;
+  const int sub = threadIdx.x & (ln - 1), step = blockDim.x / ln;
+  for (int c0 = 0; c0 < nv; c0 += step) {           // (every thread takes part in the shuffles)
+    const int c = c0 + threadIdx.x / ln;
+    float sum = 0.f;
+    if (c < nv) {
+      for (int j = first + sub; j <= p; j += ln) {
+        const int page = j / block_size, off = j - page * block_size;
+        sum += ldf(v_cache + ((int64_t)bt[page] * nv + c) * block_size + off);
+      }
+    }
+    for (int o = ln >> 1; o > 0; o >>= 1) sum += __shfl_xor(sum, o, 64);
+    if (c < nv && sub == 0) stf(pool_v + (unit * nv + c) * 8 + (b & 7), sum * inv);
   }
 }
 
@@ -85,11 +104,12 @@ __global__ __launch_bounds__(256) void qk_rows_kernel(const T* __restrict__ q, i
     const int p = (int)pos[t];
     if ((p + 1) % pool != 0) return;
     __syncthreads();                                // this workgroup's stores above are read back
-    pool_block<T>(p, block_tables + (int64_t)tseq[t] * bt_stride, k_cache, v_cache, G, d, dv, block_size, pool, pool_k, pool_v);
+    for (int half = 0; half < 2; ++half)
+      pool_block<T>(half, p, block_tables + (int64_t)tseq[t] * bt_stride, k_cache, v_cache, G, d, dv, block_size, pool, pool_k, pool_v);
   }
 }
 
-// one workgroup per token of the step: the blocks whose last token it is
+// two workgroups (keys, values) per token of the step: the block whose last token it is
 template <typename T>
 __global__ __launch_bounds__(256) void pool_blocks_kernel(const T* k_cache, const T* v_cache, int G, int d, int dv, int block_size, int pool,
                                                           const int32_t* __restrict__ slots, const int64_t* __restrict__ pos,
@@ -98,7 +118,7 @@ __global__ __launch_bounds__(256) void pool_blocks_kernel(const T* k_cache, cons
   const int64_t t = blockIdx.x;
   const int p = (int)pos[t];
   if ((p + 1) % pool != 0 || slots[t] < 0) return;
-  pool_block<T>(p, block_tables + (int64_t)tseq[t] * bt_stride, k_cache, v_cache, G, d, dv, block_size, pool, pool_k, pool_v);
+  pool_block<T>(blockIdx.y, p, block_tables + (int64_t)tseq[t] * bt_stride, k_cache, v_cache, G, d, dv, block_size, pool, pool_k, pool_v);
 }
 
 }  // namespace
@@ -130,7 +150,7 @@ extern "C" int nvs_pool_blocks(const void* k_cache, const void* v_cache, int dty
   NVS_REQUIRE(k_cache && v_cache && slots && pos && block_tables && tseq && pool_k && pool_v && n >= 0, "nvs_pool_blocks: null argument");
   NVS_REQUIRE(G > 0 && d > 0 && dv > 0 && block_size > 0 && pool > 0, "nvs_pool_blocks: G %d d %d dv %d block %d pool %d", G, d, dv, block_size, pool);
   if (n == 0) return NVS_OK;
-  NVS_DISPATCH(dtype, pool_blocks_kernel<T><<<dim3((unsigned)n), dim3(256), 0, (hipStream_t)stream>>>(
+  NVS_DISPATCH(dtype, pool_blocks_kernel<T><<<dim3((unsigned)n, 2), dim3(256), 0, (hipStream_t)stream>>>(
                           (const T*)k_cache, (const T*)v_cache, G, d, dv, block_size, pool, slots, pos, block_tables, bt_stride, tseq,
                           (T*)pool_k, (T*)pool_v));
   return nvs_check_launch("nvs_pool_blocks");

@@ -408,7 +408,7 @@ __global__ __launch_bounds__(256) void moe_gemm_tiled_kernel(const bf16_t* __res
 }
 
 // ---- combine: one workgroup per token ------------------------------------------------------------------------------------
-template <typename T>
+template <typename T, int VEC>
 __global__ void moe_combine_kernel(const T* __restrict__ rows, int64_t ldr, const int32_t* __restrict__ pair_row,
                                    const float* __restrict__ wts, int top, const T* __restrict__ h, int64_t ldh,
                                    const T* __restrict__ shared, const float* __restrict__ shared_gate, int64_t gate_stride, int width,
@@ -416,19 +416,29 @@ __global__ void moe_combine_kernel(const T* __restrict__ rows, int64_t ldr, cons
   const int64_t t = blockIdx.x;
   float sg = 0.f;
   if (shared) sg = shared_gate ? 1.f / (1.f + expf(-shared_gate[t * gate_stride])) : 1.f;      // no gate: the shared expert is added as it is
-  for (int c = threadIdx.x; c < width; c += blockDim.x) {
-    float acc = 0.f;
+  for (int c = (blockIdx.y * blockDim.x + threadIdx.x) * VEC; c < width; c += gridDim.y * blockDim.x * VEC) {
+    float acc[VEC], v[VEC];
+#pragma unroll
+    for (int i = 0; i < VEC; ++i) acc[i] = 0.f;
     for (int k = 0; k < top; ++k) {
       const int r = pair_row[t * top + k];
-      const float v = r >= 0 ? ldf(rows + (int64_t)r * ldr + c) : ldf(h + t * ldh + c);      // no row: a pass-through expert
-      acc += wts[t * top + k] * v;
+      ldv<VEC>(r >= 0 ? rows + (int64_t)r * ldr + c : h + t * ldh + c, v);      // no row: a pass-through expert
+      const float w = wts[t * top + k];
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) acc[i] += w * v[i];
     }
-    if (shared) acc += sg * ldf(shared + t * width + c);
+    if (shared) {
+      ldv<VEC>(shared + t * width + c, v);
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) acc[i] += sg * v[i];
+    }
     if (res) {                                      // the residual add is taken along: out is the new residual row, rounded
-      acc += res[t * width + c];
-      res[t * width + c] = acc;
+      ldv<VEC>(res + t * width + c, v);
+#pragma unroll
+      for (int i = 0; i < VEC; ++i) acc[i] += v[i];
+      stv<VEC>(res + t * width + c, acc);
     }
-    if (out) stf(out + t * width + c, acc);
+    if (out) stv<VEC>(out + t * width + c, acc);
   }
 }
 
@@ -534,9 +544,17 @@ extern "C" int nvs_moe_combine(const void* rows, int64_t ldr, const int32_t* pai
   NVS_REQUIRE(rows && pair_row && wts && h && (out || res) && top > 0 && width > 0 && n >= 0,
               "nvs_moe_combine: bad argument");
   if (n == 0) return NVS_OK;
-  const int threads = width >= 1024 ? 256 : (width >= 256 ? 128 : 64);
-  NVS_DISPATCH(dtype, moe_combine_kernel<T><<<dim3((unsigned)n), dim3(threads), 0, (hipStream_t)stream>>>(
-                          (const T*)rows, ldr, pair_row, wts, top, (const T*)h, ldh, (const T*)shared, shared_gate, gate_stride, width,
-                          res, (T*)out));
+  // four columns per access where every row starts aligned for it; wide rows of few tokens are spread over several workgroups
+  const uintptr_t al = (uintptr_t)rows | (uintptr_t)h | (uintptr_t)shared | (uintptr_t)res | (uintptr_t)out;
+  const bool vec = width % 4 == 0 && ldr % 4 == 0 && ldh % 4 == 0 && al % 16 == 0;
+  const int per = vec ? width / 4 : width, threads = per >= 256 ? 256 : (per >= 128 ? 128 : 64);
+  const dim3 grid((unsigned)n, n <= 512 ? (unsigned)((per + threads - 1) / threads) : 1u);
+#define NVS_COMBINE(VEC)                                                                                                              \
+  NVS_DISPATCH(dtype, moe_combine_kernel<T, VEC><<<grid, dim3(threads), 0, (hipStream_t)stream>>>(                                      \
+                          (const T*)rows, ldr, pair_row, wts, top, (const T*)h, ldh, (const T*)shared, shared_gate, gate_stride, width, \
+                          res, (T*)out))
+  if (vec) NVS_COMBINE(4);
+  else NVS_COMBINE(1);
+#undef NVS_COMBINE
   return nvs_check_launch("nvs_moe_combine");
 }

@@ -169,18 +169,68 @@ __global__ void add_group_norm_kernel(float* __restrict__ x, const T* __restrict
   }
 }
 
-// Norms on BOTH sides of a sublayer, on the 32-bit residual: the sublayer's output y[t] = a_mult * a[t] + a2_mult * a2[t] (a2 may be
-// absent) is RMS-normed with the weight (w_off + wa) and added, x[t] += rms(y[t]) * (w_off + wa); then the NEXT sublayer's input
-// out[t] = rms(x[t]) * (w_off + w). Either half may be absent (a NULL / out NULL). w_off = 1 serves weights stored as their distance
-// from one. With `rows` the kernel only reads: out[r] = norm(x[rows[r]]). One workgroup per row; all sums in 32-bit.
-template <typename T>
-__global__ void sandwich_norm_kernel(float* __restrict__ x, const T* __restrict__ a, float a_mult, const T* __restrict__ a2, float a2_mult,
-                                     const T* __restrict__ wa, const int32_t* __restrict__ rows, const T* __restrict__ w, float w_off,
-                                     int width, float eps, T* __restrict__ out) {
+// The same for ONE group without centering, four columns per access: the row stays in registers between the two passes
+// (PER accesses per thread).
+template <typename T, int PER>
+__global__ __launch_bounds__(256) void add_norm_row_kernel(float* __restrict__ x, const T* __restrict__ a, float a_mult, const float* __restrict__ b,
+                                                           const int32_t* __restrict__ rows, const T* __restrict__ w, int width, float eps,
+                                                           T* __restrict__ out) {
   __shared__ float red[16];
   const int64_t r = blockIdx.x;
   const int64_t t = rows ? (int64_t)rows[r] : r;
   float* xr = x + t * width;
+  float v[PER][4];
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int c = (i * blockDim.x + threadIdx.x) * 4;
+    if (c >= width) continue;
+    ldv<4>(xr + c, v[i]);
+    float u[4];
+    if (a) {
+      ldv<4>(a + t * width + c, u);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[i][e] += a_mult * u[e];
+    }
+    if (b) {
+      ldv<4>(b + t * width + c, u);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[i][e] += u[e];
+    }
+    if (a || b) stv<4>(xr + c, v[i]);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ss += v[i][e] * v[i][e];
+  }
+  if (!out) return;
+  const float k = w ? 1.f / sqrtf(block_sum(ss, red) / (float)width + eps) : 1.f;      // (no weights: the sum itself)
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int c = (i * blockDim.x + threadIdx.x) * 4;
+    if (c >= width) continue;
+    if (w) {
+      float u[4];
+      ldv<4>(w + c, u);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[i][e] *= k * u[e];
+    }
+    stv<4>(out + r * width + c, v[i]);
+  }
+}
+
+// Norms on BOTH sides of a sublayer, on the 32-bit residual: the sublayer's output y[t] = a_mult * a[t] + a2_mult * a2[t] (a2 may be
+// absent) is RMS-normed with the weight (w_off + wa) and added, x[t] += rms(y[t]) * (w_off + wa); then the NEXT sublayer's input
+// out[t] = rms(x[t]) * (w_off + w). Either half may be absent (a NULL / out NULL). w_off = 1 serves weights stored as their distance
+// from one. With `rows` the kernel only reads: out[r] = norm(x[rows[r]]), or with a as well out[r] = norm(x[rows[r]] + its branch), the
+// sum going to `sum`[r] instead of x. One workgroup per row; all sums in 32-bit.
+template <typename T>
+__global__ void sandwich_norm_kernel(float* __restrict__ x, const T* __restrict__ a, float a_mult, const T* __restrict__ a2, float a2_mult,
+                                     const T* __restrict__ wa, const int32_t* __restrict__ rows, const T* __restrict__ w, float w_off,
+                                     int width, float eps, float* __restrict__ sum, T* __restrict__ out) {
+  __shared__ float red[16];
+  const int64_t r = blockIdx.x;
+  const int64_t t = rows ? (int64_t)rows[r] : r;
+  const float* xi = x + t * width;
+  float* xr = rows && a ? sum + r * width : x + t * width;
   if (a) {
     float ss = 0.f;
     for (int c = threadIdx.x; c < width; c += blockDim.x) {
@@ -192,7 +242,7 @@ __global__ void sandwich_norm_kernel(float* __restrict__ x, const T* __restrict_
     for (int c = threadIdx.x; c < width; c += blockDim.x) {
       float y = a_mult * ldf(a + t * width + c);
       if (a2) y += a2_mult * ldf(a2 + t * width + c);
-      xr[c] += y * k * (w_off + ldf(wa + c));
+      xr[c] = xi[c] + y * k * (w_off + ldf(wa + c));
     }
   }
   if (!out) return;
@@ -373,6 +423,19 @@ extern "C" int nvs_add_group_norm(float* x, const void* a, float a_mult, const f
               width, groups);
   NVS_REQUIRE(!rows || (!a && !b), "nvs_add_group_norm: selected rows are only read");
   if (nrows == 0) return NVS_OK;
+  const uintptr_t al = (uintptr_t)x | (uintptr_t)a | (uintptr_t)b | (uintptr_t)w | (uintptr_t)out;
+  if (groups == 1 && !center && width % 4 == 0 && width <= 8192 && al % 16 == 0) {
+    const int per = (width + 1023) / 1024, threads = width >= 1024 ? 256 : ((width + 255) / 256) * 64;
+#define NVS_ROW(PER)                                                                                                          \
+  NVS_DISPATCH(dtype, add_norm_row_kernel<T, PER><<<dim3((unsigned)nrows), dim3(threads), 0, (hipStream_t)stream>>>(            \
+                          x, (const T*)a, a_mult, b, rows, (const T*)w, width, eps, (T*)out))
+    if (per <= 1) NVS_ROW(1);
+    else if (per <= 2) NVS_ROW(2);
+    else if (per <= 4) NVS_ROW(4);
+    else NVS_ROW(8);
+#undef NVS_ROW
+    return nvs_check_launch("nvs_add_group_norm (one group)");
+  }
   // a wavefront per group, four groups at a time; wide groups that are fewer than four are shared by 4 / groups wavefronts
   int threads = 64 * (groups < 4 ? groups : 4);
   if (groups < 4 && 4 % groups == 0 && width / groups >= 512) threads = 256;
@@ -382,12 +445,13 @@ extern "C" int nvs_add_group_norm(float* x, const void* a, float a_mult, const f
 }
 
 extern "C" int nvs_sandwich_norm(float* x, const void* a, float a_mult, const void* a2, float a2_mult, const void* wa, const int32_t* rows,
-                                 int64_t nrows, const void* w, float w_off, int dtype, int width, float eps, void* out, void* stream) {
+                                 int64_t nrows, const void* w, float w_off, int dtype, int width, float eps, float* sum, void* out,
+                                 void* stream) {
   NVS_REQUIRE(x && nrows >= 0 && width > 0 && (a || out) && (!a || wa) && (!a2 || a) && (!out || w), "nvs_sandwich_norm: bad argument (width %d)", width);
-  NVS_REQUIRE(!rows || !a, "nvs_sandwich_norm: selected rows are only read");
+  NVS_REQUIRE(!(rows && a) || sum, "nvs_sandwich_norm: selected rows are only read, their sums need a place of their own");
   if (nrows == 0) return NVS_OK;
   NVS_DISPATCH(dtype, sandwich_norm_kernel<T><<<dim3((unsigned)nrows), dim3(threads_for(width)), 0, (hipStream_t)stream>>>(
-                          x, (const T*)a, a_mult, (const T*)a2, a2_mult, (const T*)wa, rows, (const T*)w, w_off, width, eps, (T*)out));
+                          x, (const T*)a, a_mult, (const T*)a2, a2_mult, (const T*)wa, rows, (const T*)w, w_off, width, eps, sum, (T*)out));
   return nvs_check_launch("nvs_sandwich_norm");
 }
 

@@ -43,6 +43,61 @@ __global__ void causal_conv_kernel(const T* __restrict__ in, int64_t in_stride, 
   stf(out + t * channels + c, acc);
 }
 
+// Long steps: a thread takes four neighbouring channels of CONV_TB consecutive tokens with the last TAPS - 1 inputs in registers,
+// 8- or 16-byte accesses; where a portion starts, and ahead of its first token, it fetches what comes before.
+constexpr int CONV_TB = 16;
+template <typename T, typename TO, int TAPS>
+__global__ __launch_bounds__(256) void conv_tile_kernel(const T* __restrict__ in, int64_t in_stride, const T* __restrict__ w, const T* __restrict__ b,
+                                                        int channels, int act, const int32_t* __restrict__ cu_q, const int32_t* __restrict__ ctx0,
+                                                        const int32_t* __restrict__ slot, const int32_t* __restrict__ tseq, int64_t n,
+                                                        const float* __restrict__ state, TO* __restrict__ out) {
+  const int c = (blockIdx.x * blockDim.x + threadIdx.x) * 4;
+  if (c >= channels) return;
+  const int64_t t0 = (int64_t)blockIdx.y * CONV_TB, t1 = t0 + CONV_TB < n ? t0 + CONV_TB : n;
+  float wt[4][TAPS], bias[4], past[TAPS - 1][4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    bias[i] = b ? ldf(b + c + i) : 0.f;
+#pragma unroll
+    for (int k = 0; k < TAPS; ++k) wt[i][k] = ldf(w + (int64_t)(c + i) * TAPS + k);
+  }
+  int64_t q0 = 0, q1 = 0;
+  for (int64_t t = t0; t < t1; ++t) {
+    if (t >= q1) {                                  // a portion's first token, or the tile's: the inputs before it
+      const int s = tseq[t];
+      q0 = cu_q[s], q1 = cu_q[s + 1];
+      const float* tail = state + (int64_t)slot[s] * (TAPS - 1) * channels + c;
+      const bool fresh = ctx0[s] == 0;
+#pragma unroll
+      for (int k = 0; k < TAPS - 1; ++k) {
+        const int64_t back = TAPS - 1 - k, rel = t - q0 - back;      // the input `back` tokens before t, at place rel of the portion
+        if (rel >= 0) {
+          ldv<4>(in + (t - back) * in_stride + c, past[k]);
+        } else if (fresh) {
+#pragma unroll
+          for (int i = 0; i < 4; ++i) past[k][i] = 0.f;
+        } else {
+          ldv<4>(tail + (TAPS - 1 + rel) * channels, past[k]);
+        }
+      }
+    }
+    float v[4], acc[4];
+    ldv<4>(in + t * in_stride + c, v);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      acc[i] = bias[i];
+#pragma unroll
+      for (int k = 0; k < TAPS - 1; ++k) acc[i] += wt[i][k] * past[k][i];
+      acc[i] += wt[i][TAPS - 1] * v[i];
+      if (act == 1) acc[i] = siluf_(acc[i]);
+#pragma unroll
+      for (int k = 0; k + 1 < TAPS - 1; ++k) past[k][i] = past[k + 1][i];
+      past[TAPS - 2][i] = v[i];
+    }
+    stv<4>(out + t * channels + c, acc);
+  }
+}
+
 // Steps of short portions (decoding): one thread per (portion, channel) walks the portion's tokens with the last taps - 1 inputs in
 // registers and leaves them in the slot — outputs and state in one launch.
 template <typename T, typename TO, int TAPS>
@@ -549,6 +604,34 @@ __global__ void gated_group_norm_kernel(const float* __restrict__ y, const T* __
   }
 }
 
+// Norm first, then the gate, for groups of up to 256 entries: a wavefront per group, four wavefronts share a row's groups.
+template <typename T, int PER>
+__global__ __launch_bounds__(256) void norm_gate_rows_kernel(const float* __restrict__ y, const T* __restrict__ z, int64_t z_stride,
+                                                             const T* __restrict__ w, int wlen, int inner, int groups, float eps, int silu,
+                                                             const float* __restrict__ den, T* __restrict__ out) {
+  const int64_t t = blockIdx.x;
+  const int gsz = inner / groups, lane = threadIdx.x & 63;
+  for (int g = threadIdx.x >> 6; g < groups; g += 4) {
+    const int c0 = g * gsz;
+    const float dinv = den ? 1.f / den[t * groups + g] : 1.f;
+    float v[PER], gz[PER], ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int c = lane + 64 * i;
+      const bool in = c < gsz;
+      v[i] = in ? y[t * inner + c0 + c] * dinv : 0.f;
+      gz[i] = in ? ldf(z + t * z_stride + c0 + c) : 0.f;
+      ss += v[i] * v[i];
+    }
+    const float r = 1.f / sqrtf(wave_sum(ss) / (float)gsz + eps);
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int c = lane + 64 * i;
+      if (c < gsz) stf(out + t * inner + c0 + c, v[i] * r * ldf(w + (wlen < inner ? c : c0 + c)) * ((silu ? gz[i] : 1.f) / (1.f + expf(-gz[i]))));
+    }
+  }
+}
+
 }  // namespace
 
 extern "C" int nvs_causal_conv(const void* in, int64_t in_stride, int dtype, const void* w, const void* b, int channels, int taps,
@@ -578,8 +661,26 @@ extern "C" int nvs_causal_conv(const void* in, int64_t in_stride, int dtype, con
 #undef NVS_CONV_WALK
     return nvs_check_launch("nvs_causal_conv (short portions)");
   }
+  const uintptr_t al = (uintptr_t)in | (uintptr_t)out | (uintptr_t)state;
+  const bool tiles = taps >= 2 && taps <= 4 && n >= 256 && n <= 65535ll * CONV_TB && channels % 4 == 0 && in_stride % 4 == 0 && al % 16 == 0;
+  if (tiles) {
+    const dim3 grid((unsigned)((channels / 4 + 255) / 256), (unsigned)((n + CONV_TB - 1) / CONV_TB));
+#define NVS_CONV_TILE(TAPS)                                                                                                             \
+  do {                                                                                                                                  \
+    if (out_dtype == NVS_F32)                                                                                                           \
+      NVS_DISPATCH(dtype, conv_tile_kernel<T, float, TAPS><<<grid, dim3(256), 0, (hipStream_t)stream>>>(                                 \
+                              (const T*)in, in_stride, (const T*)w, (const T*)b, channels, act, cu_q, ctx0, slot, tseq, n, state, (float*)out)); \
+    else                                                                                                                                \
+      NVS_DISPATCH(dtype, conv_tile_kernel<T, T, TAPS><<<grid, dim3(256), 0, (hipStream_t)stream>>>(                                     \
+                              (const T*)in, in_stride, (const T*)w, (const T*)b, channels, act, cu_q, ctx0, slot, tseq, n, state, (T*)out)); \
+  } while (0)
+    if (taps == 2) NVS_CONV_TILE(2);
+    else if (taps == 3) NVS_CONV_TILE(3);
+    else NVS_CONV_TILE(4);
+#undef NVS_CONV_TILE
+  }
   // grid.y is limited to 65535: larger steps go in slices
-  for (int64_t t0 = 0; t0 < n; t0 += 65535) {
+  for (int64_t t0 = 0; t0 < n && !tiles; t0 += 65535) {
     const int64_t cnt = n - t0 < 65535 ? n - t0 : 65535;
     if (out_dtype == NVS_F32)
       NVS_DISPATCH(dtype, causal_conv_kernel<T, float><<<dim3(gx, (unsigned)cnt), block, 0, (hipStream_t)stream>>>(
@@ -777,6 +878,16 @@ extern "C" int nvs_gated_group_norm(const float* y, const void* z, int64_t z_str
   if (n == 0) return NVS_OK;
   NVS_REQUIRE(n <= 65535ll * 65535ll, "nvs_gated_group_norm: step too large");
   const int gsz = inner / groups;
+  if (order >= 1 && gsz <= 256 && groups >= 4) {
+#define NVS_NORM_GATE(PER)                                                                                                        \
+  NVS_DISPATCH(dtype, norm_gate_rows_kernel<T, PER><<<dim3((unsigned)n), dim3(256), 0, (hipStream_t)stream>>>(                      \
+                          y, (const T*)z, z_stride, (const T*)w, wlen, inner, groups, eps, order == 2, den, (T*)out))
+    if (gsz <= 64) NVS_NORM_GATE(1);
+    else if (gsz <= 128) NVS_NORM_GATE(2);
+    else NVS_NORM_GATE(4);
+#undef NVS_NORM_GATE
+    return nvs_check_launch("nvs_gated_group_norm (rows)");
+  }
   const dim3 block(gsz >= 1024 ? 256 : (gsz >= 128 ? 128 : 64));
   for (int64_t t0 = 0; t0 < n; t0 += 65535) {
     const int64_t cnt = n - t0 < 65535 ? n - t0 : 65535;

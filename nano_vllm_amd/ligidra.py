@@ -141,9 +141,10 @@ class LigidraForCausalLM(nn.Module):
             out.update({f"l{i}.{k}": v for k, v in layer.named_loaders().items()})
         return out
 
-    def forward(self, input_ids: torch.Tensor, positions: torch.Tensor) -> torch.Tensor:
-        """Returns the 32-bit residual stream after the last layer, [n, width]. A layer's last branch is added by the kernel that norms
-        the stream for the next layer (`pending`: the branch, and the weight of the norm on it if it has one)."""
+    def forward(self, input_ids: torch.Tensor, positions: torch.Tensor) -> tuple:
+        """Returns what compute_logits takes: the 32-bit residual stream [n, width] before the last layer's last branch, that branch, and
+        the weight of the norm on it (None: it is added as it is). A layer's last branch is always added by the kernel that norms the
+        stream next; the last one only for the rows whose logits are asked for."""
         n, cfg = input_ids.numel(), self.config
         x = torch.empty(n, cfg.hidden_size, dtype=torch.float32, device=input_ids.device)
         ops_seq.embed_norm(self.embed, input_ids, self.embed_norm, cfg.eps, x)
@@ -177,10 +178,13 @@ class LigidraForCausalLM(nn.Module):
                 if pending[0] is not None:
                     x, pending = add(x, *pending), (None, None)
                 trace.append(x.clone())
-        return add(x, *pending) if pending[0] is not None else x
+        if pending[0] is not None and pending[1] is None:
+            x, pending = add(x, *pending), (None, None)
+        return x, *pending
 
-    def compute_logits(self, x: torch.Tensor, rows: torch.Tensor | None = None, nrows: int | None = None) -> torch.Tensor:
-        """Logits of the residual rows `rows` (int32 device indices; default: each portion's last token)."""
+    def compute_logits(self, hidden: tuple, rows: torch.Tensor | None = None, nrows: int | None = None) -> torch.Tensor:
+        """Logits of the rows `rows` (int32 device indices; default: each portion's last token) of what forward() returned."""
+        x, branch, wa = hidden
         if rows is None:
             ctx = get_context()
             nrows = ctx.portions.nseq
@@ -188,7 +192,7 @@ class LigidraForCausalLM(nn.Module):
         if nrows == 0:
             return torch.empty(0, self.config.vocab_size, dtype=self.dtype, device=x.device)
         normed = torch.empty(nrows, x.shape[1], dtype=self.dtype, device=x.device)
-        ops_seq.group_norm_rows(x, rows, nrows, self.final_norm, 1, self.config.eps, normed)
+        ops_seq.offset_norm_rows(x, rows, nrows, self.final_norm, self.config.eps, normed, w_off=0.0, a=branch, wa=wa)
         return F.linear(normed, self.embed)
 
 

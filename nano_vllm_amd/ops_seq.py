@@ -26,7 +26,7 @@ SIGNATURES = {
     "nvs_scalar_norm_rows": (c_int, [_P, _P, _L, _I, _P, _I, _F, _P, _P]),
     "nvs_xielu": (c_int, [_P, _P, _F, _I, _L, _P, _P]),
     "nvs_causal_conv": (c_int, [_P, _L, _I, _P, _P, _I, _I, _I, _P, _P, _P, _P, _I, _L, _P, _P, _I, _P]),
-    "nvs_sandwich_norm": (c_int, [_P, _P, _F, _P, _F, _P, _P, _L, _P, _F, _I, _I, _F, _P, _P]),
+    "nvs_sandwich_norm": (c_int, [_P, _P, _F, _P, _F, _P, _P, _L, _P, _F, _I, _I, _F, _P, _P, _P]),
     "nvs_gated_memory_scan_workspace": (c_int64, [_I, _I, _I, _I, _L]),
     "nvs_gated_memory_scan": (c_int, [_P, _L, _L, _L, _L, _L, _L, _I, _P, _P, _F, _F, _I, _I, _I, _P, _P, _P, _I, _L, _L, _P, _P, _P, _P, _P,
                                       _L, _P]),
@@ -422,17 +422,20 @@ def sandwich_norm(x: torch.Tensor, a: torch.Tensor | None, wa: torch.Tensor | No
     assert ref is not None, "nothing to do"
     _check(lib.nvs_sandwich_norm(_ptr(x), _ptr(a), a_mult, _ptr(a2), a2_mult, _ptr(wa) if a is not None else None, None, n,
                                  _ptr(w) if out is not None else None, w_off, _same(ref, a, a2, wa if a is not None else None,
-                                                                                   w if out is not None else None, out), width, eps, _ptr(out), _stream()))
+                                                                                   w if out is not None else None, out), width, eps, None, _ptr(out), _stream()))
 
 
-def offset_norm_rows(x: torch.Tensor, rows: torch.Tensor | None, nrows: int, w: torch.Tensor, eps: float, out: torch.Tensor, w_off: float = 1.0):
-    """out[r] = rms(x[rows[r]]) * (w_off + w) (rows None: row r)."""
+def offset_norm_rows(x: torch.Tensor, rows: torch.Tensor | None, nrows: int, w: torch.Tensor, eps: float, out: torch.Tensor, w_off: float = 1.0,
+                     a: torch.Tensor | None = None, wa: torch.Tensor | None = None):
+    """out[r] = rms(x[rows[r]]) * (w_off + w) (rows None: row r); with a and wa: of x[rows[r]] + rms(a[rows[r]]) * (w_off + wa) (x stays)."""
     lib = load_library()
+    assert a is None or (rows is not None and a.shape == x.shape and a.is_contiguous() and wa.numel() == x.shape[1])
+    sums = torch.empty(nrows, x.shape[1], dtype=torch.float32, device=x.device) if a is not None else None
     assert x.dtype == torch.float32 and x.is_contiguous() and out.is_contiguous() and out.shape == (nrows, x.shape[1])
     assert rows is None or (rows.dtype == torch.int32 and rows.numel() >= nrows)
     assert rows is not None or nrows <= x.shape[0]
-    _check(lib.nvs_sandwich_norm(_ptr(x), None, 1.0, None, 1.0, None, _ptr(rows), nrows, _ptr(w), w_off, _same(out, w), x.shape[1], eps,
-                                 _ptr(out), _stream()))
+    _check(lib.nvs_sandwich_norm(_ptr(x), _ptr(a), 1.0, None, 1.0, _ptr(wa), _ptr(rows), nrows, _ptr(w), w_off, _same(out, w, a, wa), x.shape[1],
+                                 eps, _ptr(sums), _ptr(out), _stream()))
 
 
 def gated_memory_scan(proj: torch.Tensor, v_col: int, k_col: int, q_col: int, i_col: int, f_col: int, i_bias: torch.Tensor,
