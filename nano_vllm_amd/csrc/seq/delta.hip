@@ -197,12 +197,79 @@ void launch_walk(const DeltaArgs& A, int nseq, hipStream_t stream) {
 //   columns:  O = Q S | U = T (V - P), O += M U, store | S = G_C S + K^T U | P = K S of the next chunk
 //   prepare:  unit vectors, decays | decay products, G k, G q | A, M | T; K^T, G_C
 // Decay products are multiplied up (no exponential of a difference). Per-channel decays: A and M are products of G k with k / G as
-// long as no channel decays by more than 1e-20 within the chunk; otherwise every pair (j, t) is walked with the product G_t / G_j
+// long as no channel decays by more than 1e-30 within the chunk; otherwise every pair (j, t) is walked with the product G_t / G_j
 // carried along. A partial chunk is filled with tokens that change nothing (k = q = v = 0, beta = 0, decay 1).
 typedef __attribute__((ext_vector_type(4))) float f32x4_t;
 constexpr int CHUNK = 16, PREP = 256, MST = 20;      // MST: row stride of the 16 x 16 matrices in LDS (float4-aligned)
 
 __device__ __forceinline__ f32x4_t mfma4(float a, float b, f32x4_t c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
+
+// A barrier for data in LDS only: __syncthreads would also wait for every global load in flight, and the next chunk's loads are
+// meant to stay in flight across the barriers of this one.
+__device__ __forceinline__ void lds_barrier() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
+  __builtin_amdgcn_s_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
+}
+
+// softplus from the hardware exponential and logarithm; the error of the decay's exponent stays at a few 1e-8 (log(1 + e) by its
+// series where e is small)
+__device__ __forceinline__ float softplus_fast(float x) {
+  const float e = __expf(-fabsf(x));
+  return fmaxf(x, 0.f) + (e < 0.02f ? e * (1.f - e * (0.5f - e * (0.33333333f - 0.25f * e))) : __logf(1.f + e));
+}
+
+// N consecutive elements kept as they were loaded: turning them into floats waits for the load, so that is left to the use.
+template <typename T, int N>
+struct RawRun {
+  static constexpr int WORDS = N * (int)sizeof(T) / 4;
+  uint32_t w[WORDS];
+  __device__ __forceinline__ void clear() {
+#pragma unroll
+    for (int i = 0; i < WORDS; ++i) w[i] = 0u;
+  }
+  // in one piece (aligned to the piece, or to 16 bytes)
+  __device__ __forceinline__ void load(const T* p) {
+    constexpr int M = WORDS < 4 ? WORDS : 4;
+    typedef __attribute__((ext_vector_type(M))) uint32_t vec_t;
+#pragma unroll
+    for (int i = 0; i < WORDS; i += M) {
+      const vec_t f = *(const vec_t*)((const uint32_t*)p + i);
+#pragma unroll
+      for (int e = 0; e < M; ++e) w[i + e] = f[e];
+    }
+  }
+  // the first `count` elements, one at a time, zeros behind them
+  __device__ __forceinline__ void load_some(const T* p, int count) {
+    clear();
+#pragma unroll
+    for (int e = 0; e < N; ++e) {
+      if (e < count) {
+        if constexpr (sizeof(T) == 4) w[e] = __builtin_bit_cast(uint32_t, p[e]);
+        else w[e / 2] |= (uint32_t)__builtin_bit_cast(uint16_t, p[e]) << (16 * (e & 1));
+      }
+    }
+  }
+  __device__ __forceinline__ float get(int e) const {
+    if constexpr (sizeof(T) == 4) return __builtin_bit_cast(float, w[e]);
+    else return __builtin_bit_cast(float, (e & 1) ? w[e / 2] & 0xffff0000u : w[e / 2] << 16);
+  }
+};
+
+// one element, likewise
+__device__ __forceinline__ uint32_t raw_one(const float* p) { return *(const uint32_t*)p; }
+__device__ __forceinline__ uint32_t raw_one(const bf16_t* p) { return *(const uint16_t*)p; }
+template <typename T>
+__device__ __forceinline__ float raw_value(uint32_t w) { return __builtin_bit_cast(float, sizeof(T) == 4 ? w : w << 16); }
+
+// sum over the 16 lanes of a row, in every lane (rotations inside the row: plain VALU moves, no LDS)
+__device__ __forceinline__ float row16_sum(float v) {
+  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x128, 0xf, 0xf, false));      // row_ror:8
+  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x124, 0xf, 0xf, false));
+  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x122, 0xf, 0xf, false));
+  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x121, 0xf, 0xf, false));
+  return v;
+}
 
 template <int DKT, bool CH>
 struct ChunkLds {
@@ -215,7 +282,7 @@ struct ChunkLds {
   float gc[DKP];                                    // G_C
   float part[4][CHUNK][MST];                        // A (0, 1) and M (2, 3) in two halves of the channels each
   float ratio[CH ? 1 : CHUNK][MST];                 // G_t / G_j of per-head decays
-  float T[CHUNK][MST], M[CHUNK][MST], L[CHUNK][MST];
+  float T[CHUNK][MST], M[CHUNK][MST];
   float beta[CHUNK];
   int strong;                                       // chunk number + 1 of the last chunk with a channel below the limit
 };
@@ -235,7 +302,7 @@ __global__ __launch_bounds__(768) void delta_chunk_kernel(const DeltaArgs A) {
   const int nch = (int)((q1 - q0 + CHUNK - 1) / CHUNK);
   if (tid == 0) W.strong = 0;
 
-  // ---- prepare: thread (token pt, lane pl of 16) holds channels pl + 16 e of its token
+  // ---- prepare: thread (token pt, lane pl of 16) holds the DKT channels from pl DKT on of its token
   const int pt = (tid >> 4) & 15, pl = tid & 15;
   const T* qp = (const T*)A.qkv + (int64_t)grp * dk;
   const T* kp = (const T*)A.qkv + (int64_t)(A.G + grp) * dk;
@@ -243,39 +310,51 @@ __global__ __launch_bounds__(768) void delta_chunk_kernel(const DeltaArgs A) {
   const T* bp = (const T*)A.gates + A.b_col + h;
   const float* dtb = A.dt_bias + (CH ? (int64_t)h * dk : h);
   const float rate = -expf(A.A_log[h]);
-  float rk_[DKT], rq_[DKT], ra_[CH ? DKT : 1], rb = 0.f;
+  RawRun<T, DKT> rk_, rq_, ra_;                     // (ra_: per-channel decays only)
+  uint32_t ra1 = 0u, rb = 0u;
+  const int64_t rows_al = A.qkv_stride | dk | (CH ? A.decays_stride | A.a_col : 0);
+  const bool runs = rows_al % DKT == 0 && ((uintptr_t)A.qkv | (uintptr_t)(CH ? A.decays : A.qkv)) % 16 == 0;      // whole runs, aligned
+  const int pc = pl * DKT;
+  float dtc[CH ? DKT : 1];
+  if (CH) {
+#pragma unroll
+    for (int e = 0; e < DKT; ++e) dtc[e] = pc + e < dk ? dtb[pc + e] : 0.f;
+  } else {
+    dtc[0] = dtb[0];
+  }
   auto load = [&](int n) {
     const int64_t t = q0 + (int64_t)n * CHUNK + pt;
     const bool in = t < q1;
-#pragma unroll
-    for (int e = 0; e < DKT; ++e) {
-      const int c = pl + 16 * e;
-      const bool ok = in && c < dk;
-      rk_[e] = ok ? ldf(kp + t * A.qkv_stride + c) : 0.f;
-      rq_[e] = ok ? ldf(qp + t * A.qkv_stride + c) : 0.f;
-      if (CH) ra_[e] = ok ? ldf(ap + t * A.decays_stride + c) : 0.f;
+    if (in && runs && pc < dk) {
+      rk_.load(kp + t * A.qkv_stride + pc);
+      rq_.load(qp + t * A.qkv_stride + pc);
+      if constexpr (CH) ra_.load(ap + t * A.decays_stride + pc);
+    } else {
+      const int count = in && !runs ? dk - pc : 0;
+      rk_.load_some(kp + t * A.qkv_stride + pc, count);
+      rq_.load_some(qp + t * A.qkv_stride + pc, count);
+      if constexpr (CH) ra_.load_some(ap + t * A.decays_stride + pc, count);
     }
-    if (!CH) ra_[0] = in ? ldf(ap + t * A.gates_stride) : 0.f;
-    rb = in ? ldf(bp + t * A.gates_stride) : 0.f;
+    if (in) {
+      rb = raw_one(bp + t * A.gates_stride);
+      if constexpr (!CH) ra1 = raw_one(ap + t * A.gates_stride);
+    }
   };
   auto stage = [&](int n) {
     const bool in = q0 + (int64_t)n * CHUNK + pt < q1;
     float sk = 0.f, sq = 0.f;
 #pragma unroll
-    for (int e = 0; e < DKT; ++e) sk += rk_[e] * rk_[e], sq += rq_[e] * rq_[e];
-#pragma unroll
-    for (int o = 8; o > 0; o >>= 1) sk += __shfl_xor(sk, o, 64), sq += __shfl_xor(sq, o, 64);
-    const float fk = 1.f / sqrtf(sk + UNIT_EPS), fq = A.q_scale / sqrtf(sq + UNIT_EPS);
+    for (int e = 0; e < DKT; ++e) sk += rk_.get(e) * rk_.get(e), sq += rq_.get(e) * rq_.get(e);
+    const float fk = 1.f / sqrtf(row16_sum(sk) + UNIT_EPS), fq = A.q_scale / sqrtf(row16_sum(sq) + UNIT_EPS);
 #pragma unroll
     for (int e = 0; e < DKT; ++e) {
-      const int c = pl + 16 * e;
-      W.kn[pt][c] = rk_[e] * fk;
-      W.qn[pt][c] = rq_[e] * fq;
-      if (CH) W.g[pt][c] = in && c < dk ? expf(rate * softplusf_(ra_[e] + dtb[c < dk ? c : 0])) : 1.f;
+      W.kn[pt][pc + e] = rk_.get(e) * fk;
+      W.qn[pt][pc + e] = rq_.get(e) * fq;
+      if constexpr (CH) W.g[pt][pc + e] = in && pc + e < dk ? __expf(rate * softplus_fast(ra_.get(e) + dtc[e])) : 1.f;
     }
     if (pl == 0) {
-      if (!CH) W.g[0][pt] = in ? expf(rate * softplusf_(ra_[0] + dtb[0])) : 1.f;
-      W.beta[pt] = in ? 1.f / (1.f + expf(-rb)) : 0.f;
+      if constexpr (!CH) W.g[0][pt] = in ? __expf(rate * softplus_fast(raw_value<T>(ra1) + dtc[0])) : 1.f;
+      W.beta[pt] = in ? 1.f / (1.f + __expf(-raw_value<T>(rb))) : 0.f;
     }
   };
   auto products = [&](int n) {                       // G k, G q, k / G: a channel per thread, K and Q parts apart
@@ -288,9 +367,9 @@ __global__ __launch_bounds__(768) void delta_chunk_kernel(const DeltaArgs A) {
           G *= CH ? W.g[t][c] : W.g[0][t];
           const float k = W.kn[t][c];
           W.kg[t][c] = G * k;
-          if (CH) W.ki[t][c] = k / G;
+          if (CH) W.ki[t][c] = k * __builtin_amdgcn_rcpf(G);
         }
-        if (CH && G < 1e-20f) W.strong = n + 1;
+        if (CH && G < 1e-30f) W.strong = n + 1;
       } else {
 #pragma unroll
         for (int t = 0; t < CHUNK; ++t) {
@@ -301,29 +380,27 @@ __global__ __launch_bounds__(768) void delta_chunk_kernel(const DeltaArgs A) {
     }
     if (!CH) {
       float r = 1.f;
-      for (int i = pl + 1; i <= pt; ++i) r *= W.g[0][i];
+#pragma unroll
+      for (int i = 1; i < CHUNK; ++i) r *= i > pl && i <= pt ? W.g[0][i] : 1.f;
       W.ratio[pt][pl] = r;
     }
   };
   auto matrices = [&](int n) {
     if (CH && W.strong == n + 1) {
-      // pair by pair: thread (token j = pt, lane pl) carries k_j times the decays since j through the later tokens
+      // pair by pair: thread (token j = pt, lane pl) carries its channels of k_j times the decays since j through the later tokens
       float w[DKT];
 #pragma unroll
-      for (int e = 0; e < DKT; ++e) w[e] = W.kn[pt][pl + 16 * e];
+      for (int e = 0; e < DKT; ++e) w[e] = W.kn[pt][pc + e];
+#pragma unroll 4
       for (int t = 0; t < CHUNK; ++t) {
         float a = 0.f, m = 0.f;
-        if (t >= pt) {
 #pragma unroll
-          for (int e = 0; e < DKT; ++e) {
-            const int c = pl + 16 * e;
-            if (t > pt) w[e] *= W.g[t][c];
-            a += W.kn[t][c] * w[e];
-            m += W.qn[t][c] * w[e];
-          }
+        for (int e = 0; e < DKT; ++e) {
+          w[e] *= t > pt ? W.g[t][pc + e] : 1.f;
+          a += W.kn[t][pc + e] * w[e];
+          m += W.qn[t][pc + e] * w[e];
         }
-#pragma unroll
-        for (int o = 8; o > 0; o >>= 1) a += __shfl_xor(a, o, 64), m += __shfl_xor(m, o, 64);
+        a = row16_sum(a), m = row16_sum(m);          // (entries above the diagonal are not looked at)
         if (pl == 0) W.part[0][t][pt] = a, W.part[1][t][pt] = 0.f, W.part[2][t][pt] = m, W.part[3][t][pt] = 0.f;
       }
       return;
@@ -348,36 +425,57 @@ __global__ __launch_bounds__(768) void delta_chunk_kernel(const DeltaArgs A) {
   };
   auto solve = [&]() {
     if (wave == 0) {
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {                  // L = beta A below the diagonal
-        const int t = 4 * i + lq;
-        float a = W.part[0][t][li] + W.part[1][t][li];
-        if (!CH) a *= W.ratio[t][li];
-        W.L[t][li] = li < t ? W.beta[t] * a : 0.f;
+      // T = (I + L)^-1, L = beta A below the diagonal, by doubling the blocks whose inverses are known: with T block diagonal (blocks
+      // of b) and L_b the entries of L that couple the two halves of a block of 2 b, T <- T - T L_b T. L stays in registers as
+      // an A operand; X = L_b T comes out as the B operand that T X needs; T goes through LDS once per step to become an A operand.
+      const float4 a0 = *(const float4*)&W.part[0][li][4 * lq], a1 = *(const float4*)&W.part[1][li][4 * lq];
+      const float bt = W.beta[li];
+      float L[4] = {a0.x + a1.x, a0.y + a1.y, a0.z + a1.z, a0.w + a1.w};
+      if (!CH) {
+        const float4 r = *(const float4*)&W.ratio[li][4 * lq];
+        L[0] *= r.x, L[1] *= r.y, L[2] *= r.z, L[3] *= r.w;
       }
-      __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "workgroup");
-      __builtin_amdgcn_wave_barrier();
-      float x[CHUNK];                                // column li of (I + L)^-1, row after row
+      f32x4_t Tm;
 #pragma unroll
-      for (int t = 0; t < CHUNK; ++t) {
-        float v = t == li ? 1.f : 0.f;
+      for (int r = 0; r < 4; ++r) Tm[r] = 4 * lq + r == li ? 1.f : 0.f;
 #pragma unroll
-        for (int j = 0; j < t; ++j) v -= W.L[t][j] * x[j];
-        x[t] = v;
+      for (int b = 1; b < CHUNK; b *= 2) {
+        if (b > 1) {
+#pragma unroll
+          for (int r = 0; r < 4; ++r) W.T[4 * lq + r][li] = Tm[r];
+          __builtin_amdgcn_fence(__ATOMIC_ACQ_REL, "workgroup", "local");
+          __builtin_amdgcn_wave_barrier();
+        }
+        f32x4_t X = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int k = 4 * lq + r;                  // entry (li, k): below the diagonal, other half of the same block of 2 b
+          const bool couples = li / (2 * b) == k / (2 * b) && (li & b) && !(k & b);
+          X = mfma4(couples ? bt * L[r] : 0.f, Tm[r], X);
+        }
+        if (b == 1) {                                // (T is the unit matrix)
+          Tm -= X;
+        } else {
+          const float4 t4 = *(const float4*)&W.T[li][4 * lq];
+          Tm = mfma4(-t4.x, X[0], Tm);
+          Tm = mfma4(-t4.y, X[1], Tm);
+          Tm = mfma4(-t4.z, X[2], Tm);
+          Tm = mfma4(-t4.w, X[3], Tm);
+          __builtin_amdgcn_wave_barrier();
+        }
       }
-      const float b = W.beta[li];
-      if (lq == 0) {
 #pragma unroll
-        for (int t = 0; t < CHUNK; ++t) W.T[t][li] = x[t] * b;
-      }
+      for (int r = 0; r < 4; ++r) W.T[4 * lq + r][li] = Tm[r] * bt;      // times beta of the column: U = T diag(beta) (V - P)
     } else if (wave == 1) {
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int t = 4 * i + lq;
-        float m = W.part[2][t][li] + W.part[3][t][li];
-        if (!CH) m *= W.ratio[t][li];
-        W.M[t][li] = li <= t ? m : 0.f;
+      const float4 m0 = *(const float4*)&W.part[2][li][4 * lq], m1 = *(const float4*)&W.part[3][li][4 * lq];
+      float m[4] = {m0.x + m1.x, m0.y + m1.y, m0.z + m1.z, m0.w + m1.w};
+      if (!CH) {
+        const float4 r = *(const float4*)&W.ratio[li][4 * lq];
+        m[0] *= r.x, m[1] *= r.y, m[2] *= r.z, m[3] *= r.w;
       }
+#pragma unroll
+      for (int r = 0; r < 4; ++r) m[r] = 4 * lq + r <= li ? m[r] : 0.f;
+      *(float4*)&W.M[li][4 * lq] = make_float4(m[0], m[1], m[2], m[3]);
     } else {
       for (int c = tid - 128; c < DKP; c += 128) {
         float D = 1.f, col[CHUNK];
@@ -396,20 +494,20 @@ __global__ __launch_bounds__(768) void delta_chunk_kernel(const DeltaArgs A) {
   // the two roles in loops of their own (their registers are then not live together); both meet in the same 1 + 4 (nch + 1) barriers
   if (prep) {
     load(0);
-    __syncthreads();
+    lds_barrier();
     for (int n = 0; n <= nch; ++n) {                // chunk n is prepared while chunk n - 1 is worked on
       const bool next = n < nch;
       if (next) {
         stage(n);
         if (n + 1 < nch) load(n + 1);
       }
-      __syncthreads();
+      lds_barrier();
       if (next) products(n);
-      __syncthreads();
+      lds_barrier();
       if (next) matrices(n);
-      __syncthreads();
+      lds_barrier();
       if (next) solve();
-      __syncthreads();
+      lds_barrier();
     }
     return;
   }
@@ -419,7 +517,7 @@ __global__ __launch_bounds__(768) void delta_chunk_kernel(const DeltaArgs A) {
   float* Sc = A.S + (((int64_t)A.slot[s] * A.heads + h) * dv + (own ? col : 0)) * dk;
   const T* vp = (const T*)A.qkv + (int64_t)2 * A.G * dk + (int64_t)h * dv + col;
   f32x4_t st[DKT], P = {0.f, 0.f, 0.f, 0.f}, O = {0.f, 0.f, 0.f, 0.f}, U = {0.f, 0.f, 0.f, 0.f};
-  float v[4] = {0.f, 0.f, 0.f, 0.f};
+  uint32_t v[4] = {0u, 0u, 0u, 0u};                 // (raw: see RawRun)
 #pragma unroll
   for (int i = 0; i < DKT; ++i) st[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
   if (own && A.ctx0[s] != 0) {
@@ -439,7 +537,7 @@ __global__ __launch_bounds__(768) void delta_chunk_kernel(const DeltaArgs A) {
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int64_t t = q0 + (int64_t)n * CHUNK + 4 * lq + r;
-      v[r] = own && t < q1 ? ldf(vp + t * A.qkv_stride) : 0.f;
+      v[r] = own && t < q1 ? raw_one(vp + t * A.qkv_stride) : 0u;
     }
   };
   auto times_state = [&](const float (&m)[CHUNK][Lds::LD]) {      // m S, [16 tokens x 16 columns]
@@ -455,15 +553,15 @@ __global__ __launch_bounds__(768) void delta_chunk_kernel(const DeltaArgs A) {
     return a0 + a1;
   };
   load_v(0);
-  __syncthreads();
+  lds_barrier();
   for (int n = -1; n < nch; ++n) {
     const bool next = n + 1 < nch;
     if (n >= 0) O = times_state(W.qg);
-    __syncthreads();
+    lds_barrier();
     if (n >= 0) {
       f32x4_t X;
 #pragma unroll
-      for (int r = 0; r < 4; ++r) X[r] = v[r] - P[r];
+      for (int r = 0; r < 4; ++r) X[r] = raw_value<T>(v[r]) - P[r];
       if (next) load_v(n + 1);
       const float4 t4 = *(const float4*)&W.T[li][4 * lq], m4 = *(const float4*)&W.M[li][4 * lq];
       U = mfma4(t4.x, X[0], f32x4_t{0.f, 0.f, 0.f, 0.f});
@@ -482,7 +580,7 @@ __global__ __launch_bounds__(768) void delta_chunk_kernel(const DeltaArgs A) {
         }
       }
     }
-    __syncthreads();
+    lds_barrier();
     if (n >= 0) {
 #pragma unroll
       for (int i = 0; i < DKT; ++i) {
@@ -494,9 +592,9 @@ __global__ __launch_bounds__(768) void delta_chunk_kernel(const DeltaArgs A) {
         st[i] = mfma4(a.w, U[3], st[i]);
       }
     }
-    __syncthreads();
+    lds_barrier();
     if (next) P = times_state(W.kg);
-    __syncthreads();
+    lds_barrier();
   }
   if (own) {
 #pragma unroll
