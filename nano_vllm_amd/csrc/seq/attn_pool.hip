@@ -35,17 +35,23 @@ __device__ void pool_block(int half, int p, const int32_t* __restrict__ bt, cons
   int ln = 1;
   while (ln < pool && ln < 16) ln <<= 1;
   const int sub = threadIdx.x & (ln - 1), step = blockDim.x / ln;
-  for (int c0 = 0; c0 < nv; c0 += step) {           // (every thread takes part in the shuffles)
-    const int c = c0 + threadIdx.x / ln;
-    float sum = 0.f;
-    if (c < nv) {
-      for (int j = first + sub; j <= p; j += ln) {
-        const int page = j / block_size, off = j - page * block_size;
-        sum += ldf(v_cache + ((int64_t)bt[page] * nv + c) * block_size + off);
-      }
+  for (int c0 = threadIdx.x / ln; c0 - (int)(threadIdx.x / ln) < nv; c0 += 8 * step) {      // (every thread takes part in the shuffles)
+    float sum[8];
+#pragma unroll
+    for (int u = 0; u < 8; ++u) sum[u] = 0.f;
+    for (int j = first + sub; j <= p; j += ln) {
+      const int page = j / block_size, off = j - page * block_size;
+      const T* src = v_cache + ((int64_t)bt[page] * nv + c0) * block_size + off;
+#pragma unroll
+      for (int u = 0; u < 8; ++u)
+        if (c0 + u * step < nv) sum[u] += ldf(src + (int64_t)u * step * block_size);
     }
-    for (int o = ln >> 1; o > 0; o >>= 1) sum += __shfl_xor(sum, o, 64);
-    if (c < nv && sub == 0) stf(pool_v + (unit * nv + c) * 8 + (b & 7), sum * inv);
+#pragma unroll
+    for (int u = 0; u < 8; ++u) {
+      for (int o = ln >> 1; o > 0; o >>= 1) sum[u] += __shfl_xor(sum[u], o, 64);
+      const int c = c0 + u * step;
+      if (c < nv && sub == 0) stf(pool_v + (unit * nv + c) * 8 + (b & 7), sum[u] * inv);
+    }
   }
 }
 
@@ -53,7 +59,7 @@ __device__ void pool_block(int half, int p, const int32_t* __restrict__ bt, cons
 // its weights, rotated per head, and the value row into the paged cache. finish: the step brings one token per sequence, so a
 // block that this token completes has all its other tokens in the cache already and its mean is taken here.
 template <typename T>
-__global__ __launch_bounds__(256) void qk_rows_kernel(const T* __restrict__ q, int64_t q_stride, int q_cols, const T* __restrict__ k,
+__global__ __launch_bounds__(256) void qk_rows_kernel(const T* __restrict__ q, int64_t q_stride, int q_cols, int q_vec, const T* __restrict__ k,
                                                       const T* __restrict__ v, int64_t stride, const T* __restrict__ knorm, float eps, int G,
                                                       int d, int dv, int block_size, const int32_t* __restrict__ slots,
                                                       const int64_t* __restrict__ pos, const float* __restrict__ rot_freq, int rot_dims,
@@ -63,9 +69,17 @@ __global__ __launch_bounds__(256) void qk_rows_kernel(const T* __restrict__ q, i
   __shared__ float red[16];
   const int64_t t = blockIdx.x;
   float ss = 0.f;
-  for (int c = threadIdx.x; c < q_cols; c += blockDim.x) {
-    const float x = ldf(q + t * q_stride + c);
-    ss += x * x;
+  if (q_vec) {
+    for (int c = threadIdx.x * 4; c < q_cols; c += blockDim.x * 4) {
+      float x[4];
+      ldv<4>(q + t * q_stride + c, x);
+      ss += x[0] * x[0] + x[1] * x[1] + x[2] * x[2] + x[3] * x[3];
+    }
+  } else {
+    for (int c = threadIdx.x; c < q_cols; c += blockDim.x) {
+      const float x = ldf(q + t * q_stride + c);
+      ss += x * x;
+    }
   }
   ss = block_sum(ss, red);
   if (threadIdx.x == 0) q_row[t] = 1.f / sqrtf(ss / (float)q_cols + eps);
@@ -109,13 +123,17 @@ __global__ __launch_bounds__(256) void qk_rows_kernel(const T* __restrict__ q, i
   }
 }
 
-// two workgroups (keys, values) per token of the step: the block whose last token it is
+// Two workgroups (keys, values) per token of the step: the block whose last token it is. Workgroups are dealt to the eight XCDs in
+// turn and the tokens that end a block are `pool` apart, so tokens are dealt to workgroups in strides of `pool` (`runs` of them):
+// neighbouring workgroups then hold the ends of neighbouring blocks, and not one XCD all of them.
 template <typename T>
 __global__ __launch_bounds__(256) void pool_blocks_kernel(const T* k_cache, const T* v_cache, int G, int d, int dv, int block_size, int pool,
+                                                          int64_t n, unsigned runs,
                                                           const int32_t* __restrict__ slots, const int64_t* __restrict__ pos,
                                                           const int32_t* __restrict__ block_tables, int64_t bt_stride,
                                                           const int32_t* __restrict__ tseq, T* pool_k, T* pool_v) {
-  const int64_t t = blockIdx.x;
+  const int64_t t = (int64_t)(blockIdx.x % runs) * pool + blockIdx.x / runs;
+  if (t >= n) return;
   const int p = (int)pos[t];
   if ((p + 1) % pool != 0 || slots[t] < 0) return;
   pool_block<T>(blockIdx.y, p, block_tables + (int64_t)tseq[t] * bt_stride, k_cache, v_cache, G, d, dv, block_size, pool, pool_k, pool_v);
@@ -137,8 +155,9 @@ extern "C" int nvs_qk_rows(const void* q, int64_t q_stride, int q_cols, const vo
               "nvs_qk_rows: G %d d %d dv %d block %d rotation %d", G, d, dv, block_size, rot_dims);
   NVS_REQUIRE(pool >= 0 && (!(k && pool > 0 && finish) || (block_tables && tseq && pool_k && pool_v)), "nvs_qk_rows: pooled blocks (%d) without their tensors", pool);
   if (n == 0) return NVS_OK;
+  const int q_vec = q_cols % 4 == 0 && q_stride % 4 == 0 && (uintptr_t)q % 16 == 0;
   NVS_DISPATCH(dtype, qk_rows_kernel<T><<<dim3((unsigned)n), dim3(256), 0, (hipStream_t)stream>>>(
-                          (const T*)q, q_stride, q_cols, (const T*)k, (const T*)v, stride, (const T*)knorm, eps, G, d, dv, block_size, slots, pos,
+                          (const T*)q, q_stride, q_cols, q_vec, (const T*)k, (const T*)v, stride, (const T*)knorm, eps, G, d, dv, block_size, slots, pos,
                           rot_freq, rot_dims, q_row, (T*)k_cache, (T*)v_cache, pool, finish, block_tables, bt_stride, tseq, (T*)pool_k,
                           (T*)pool_v));
   return nvs_check_launch("nvs_qk_rows");
@@ -150,8 +169,10 @@ extern "C" int nvs_pool_blocks(const void* k_cache, const void* v_cache, int dty
   NVS_REQUIRE(k_cache && v_cache && slots && pos && block_tables && tseq && pool_k && pool_v && n >= 0, "nvs_pool_blocks: null argument");
   NVS_REQUIRE(G > 0 && d > 0 && dv > 0 && block_size > 0 && pool > 0, "nvs_pool_blocks: G %d d %d dv %d block %d pool %d", G, d, dv, block_size, pool);
   if (n == 0) return NVS_OK;
-  NVS_DISPATCH(dtype, pool_blocks_kernel<T><<<dim3((unsigned)n, 2), dim3(256), 0, (hipStream_t)stream>>>(
-                          (const T*)k_cache, (const T*)v_cache, G, d, dv, block_size, pool, slots, pos, block_tables, bt_stride, tseq,
+  const int64_t runs = (n + pool - 1) / pool;
+  NVS_REQUIRE(runs * pool < (1ll << 31), "nvs_pool_blocks: step too large");
+  NVS_DISPATCH(dtype, pool_blocks_kernel<T><<<dim3((unsigned)(runs * pool), 2), dim3(256), 0, (hipStream_t)stream>>>(
+                          (const T*)k_cache, (const T*)v_cache, G, d, dv, block_size, pool, n, (unsigned)runs, slots, pos, block_tables, bt_stride, tseq,
                           (T*)pool_k, (T*)pool_v));
   return nvs_check_launch("nvs_pool_blocks");
 }

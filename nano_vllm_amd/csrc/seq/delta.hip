@@ -614,10 +614,11 @@ __global__ __launch_bounds__(768) void delta_chunk_kernel(const DeltaArgs A) {
 template <typename T, int DKT, bool CH>
 void launch_chunk_size(const DeltaArgs& A, int nseq, hipStream_t stream) {
   const int tiles = (A.dv + 15) / 16;
-  // column wavefronts per workgroup: all columns of a head together (they share the preparation) once the (portion, head) pairs
-  // fill the chip, fewer columns per workgroup otherwise
+  // column wavefronts per workgroup: all columns of a head together (they share the preparation, which bounds a chunk's time), fewer
+  // of them while the workgroups do not even fill half the chip (measured, 128 x 128 heads, 2,048 tokens: 256 pairs 780 us with 8
+  // wavefronts, 900 with 4, 1,690 with 2; 64 pairs 770 / 590 / 580)
   int ncw = tiles < 8 ? tiles : 8;
-  while (ncw > 1 && (int64_t)A.heads * nseq * ((tiles + ncw - 1) / ncw) < 384) ncw = (ncw + 1) / 2;
+  while (ncw > 1 && (int64_t)A.heads * nseq * ((tiles + ncw - 1) / ncw) < 128) ncw = (ncw + 1) / 2;
   const size_t lds = sizeof(ChunkLds<DKT, CH>);
   if (lds > 48 * 1024) (void)hipFuncSetAttribute((const void*)delta_chunk_kernel<T, DKT, CH>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
   delta_chunk_kernel<T, DKT, CH><<<dim3(A.heads, (unsigned)nseq, (unsigned)((tiles + ncw - 1) / ncw)), dim3(64 * (4 + ncw)), lds, stream>>>(A);

@@ -255,7 +255,98 @@ __global__ void sandwich_norm_kernel(float* __restrict__ x, const T* __restrict_
   for (int c = threadIdx.x; c < width; c += blockDim.x) stf(out + r * width + c, xr[c] * k * (w_off + ldf(w + c)));
 }
 
-// x[t] = rms(table[ids[t]]) * w: one workgroup per token
+// The same with the rows in registers, four columns per access (PER accesses per thread).
+template <typename T, int PER>
+__global__ __launch_bounds__(256) void sandwich_row_kernel(float* __restrict__ x, const T* __restrict__ a, float a_mult, const T* __restrict__ a2,
+                                                           float a2_mult, const T* __restrict__ wa, const int32_t* __restrict__ rows,
+                                                           const T* __restrict__ w, float w_off, int width, float eps, T* __restrict__ out) {
+  __shared__ float red[16];
+  const int64_t r = blockIdx.x;
+  const int64_t t = rows ? (int64_t)rows[r] : r;
+  float v[PER][4];
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int c = (i * blockDim.x + threadIdx.x) * 4;
+    if (c < width) ldv<4>(x + t * width + c, v[i]);
+  }
+  if (a) {
+    float y[PER][4], ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int c = (i * blockDim.x + threadIdx.x) * 4;
+      if (c >= width) continue;
+      ldv<4>(a + t * width + c, y[i]);
+      float u[4] = {0.f, 0.f, 0.f, 0.f};
+      if (a2) ldv<4>(a2 + t * width + c, u);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        y[i][e] = a_mult * y[i][e] + a2_mult * u[e];
+        ss += y[i][e] * y[i][e];
+      }
+    }
+    const float k = 1.f / sqrtf(block_sum(ss, red) / (float)width + eps);
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int c = (i * blockDim.x + threadIdx.x) * 4;
+      if (c >= width) continue;
+      float u[4];
+      ldv<4>(wa + c, u);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) v[i][e] += y[i][e] * k * (w_off + u[e]);
+      if (!rows) stv<4>(x + t * width + c, v[i]);   // (selected rows are only read)
+    }
+  }
+  if (!out) return;
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    if ((int)(i * blockDim.x + threadIdx.x) * 4 >= width) continue;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ss += v[i][e] * v[i][e];
+  }
+  const float k = 1.f / sqrtf(block_sum(ss, red) / (float)width + eps);
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int c = (i * blockDim.x + threadIdx.x) * 4;
+    if (c >= width) continue;
+    float u[4];
+    ldv<4>(w + c, u);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[i][e] *= k * (w_off + u[e]);
+    stv<4>(out + r * width + c, v[i]);
+  }
+}
+
+// x[t] = rms(table[ids[t]]) * w: one workgroup per token, the row in registers (PER accesses of four columns per thread)
+template <typename T, int PER>
+__global__ __launch_bounds__(256) void embed_norm_row_kernel(const T* __restrict__ table, const int64_t* __restrict__ ids, int width,
+                                                             const T* __restrict__ w, float eps, float* __restrict__ x) {
+  __shared__ float red[16];
+  const int64_t t = blockIdx.x;
+  const T* row = table + ids[t] * width;
+  float v[PER][4], ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int c = (i * blockDim.x + threadIdx.x) * 4;
+    if (c >= width) continue;
+    ldv<4>(row + c, v[i]);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ss += v[i][e] * v[i][e];
+  }
+  const float k = 1.f / sqrtf(block_sum(ss, red) / (float)width + eps);
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int c = (i * blockDim.x + threadIdx.x) * 4;
+    if (c >= width) continue;
+    float u[4];
+    ldv<4>(w + c, u);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[i][e] *= k * u[e];
+    stv<4>(x + t * width + c, v[i]);
+  }
+}
+
+// the same for any width
 template <typename T>
 __global__ void embed_norm_kernel(const T* __restrict__ table, const int64_t* __restrict__ ids, int width, const T* __restrict__ w, float eps,
                                   float* __restrict__ x) {
@@ -376,6 +467,21 @@ __global__ void scale_softcap_kernel(const T* __restrict__ in, float scale, floa
   }
 }
 
+// row kernels: threads and accesses of four columns per thread (1, 2, 4 or 8; 0: the row does not fit or is not aligned for them)
+int row_plan(int width, uintptr_t al, int* threads) {
+  if (width % 4 || width > 8192 || al % 16) return 0;
+  *threads = width >= 1024 ? 256 : ((width + 255) / 256) * 64;
+  const int per = (width + 1023) / 1024;
+  return per <= 1 ? 1 : (per <= 2 ? 2 : (per <= 4 ? 4 : 8));
+}
+#define NVS_ROW_CASES(per, NAME) \
+  switch (per) {                 \
+    case 1: NAME(1); break;      \
+    case 2: NAME(2); break;      \
+    case 4: NAME(4); break;      \
+    default: NAME(8);            \
+  }
+
 int threads_for(int width) { return width >= 1024 ? 256 : (width >= 256 ? 128 : 64); }
 
 }  // namespace
@@ -424,15 +530,13 @@ extern "C" int nvs_add_group_norm(float* x, const void* a, float a_mult, const f
   NVS_REQUIRE(!rows || (!a && !b), "nvs_add_group_norm: selected rows are only read");
   if (nrows == 0) return NVS_OK;
   const uintptr_t al = (uintptr_t)x | (uintptr_t)a | (uintptr_t)b | (uintptr_t)w | (uintptr_t)out;
-  if (groups == 1 && !center && width % 4 == 0 && width <= 8192 && al % 16 == 0) {
-    const int per = (width + 1023) / 1024, threads = width >= 1024 ? 256 : ((width + 255) / 256) * 64;
-#define NVS_ROW(PER)                                                                                                          \
-  NVS_DISPATCH(dtype, add_norm_row_kernel<T, PER><<<dim3((unsigned)nrows), dim3(threads), 0, (hipStream_t)stream>>>(            \
+  int row_threads = 0;
+  const int per = groups == 1 && !center ? row_plan(width, al, &row_threads) : 0;
+  if (per) {
+#define NVS_ROW(PER)                                                                                                           \
+  NVS_DISPATCH(dtype, add_norm_row_kernel<T, PER><<<dim3((unsigned)nrows), dim3(row_threads), 0, (hipStream_t)stream>>>(         \
                           x, (const T*)a, a_mult, b, rows, (const T*)w, width, eps, (T*)out))
-    if (per <= 1) NVS_ROW(1);
-    else if (per <= 2) NVS_ROW(2);
-    else if (per <= 4) NVS_ROW(4);
-    else NVS_ROW(8);
+    NVS_ROW_CASES(per, NVS_ROW)
 #undef NVS_ROW
     return nvs_check_launch("nvs_add_group_norm (one group)");
   }
@@ -450,6 +554,16 @@ extern "C" int nvs_sandwich_norm(float* x, const void* a, float a_mult, const vo
   NVS_REQUIRE(x && nrows >= 0 && width > 0 && (a || out) && (!a || wa) && (!a2 || a) && (!out || w), "nvs_sandwich_norm: bad argument (width %d)", width);
   NVS_REQUIRE(!(rows && a) || sum, "nvs_sandwich_norm: selected rows are only read, their sums need a place of their own");
   if (nrows == 0) return NVS_OK;
+  int row_threads = 0;
+  const int per = row_plan(width, (uintptr_t)x | (uintptr_t)a | (uintptr_t)a2 | (uintptr_t)wa | (uintptr_t)w | (uintptr_t)out, &row_threads);
+  if (per) {
+#define NVS_ROW(PER)                                                                                                           \
+  NVS_DISPATCH(dtype, sandwich_row_kernel<T, PER><<<dim3((unsigned)nrows), dim3(row_threads), 0, (hipStream_t)stream>>>(         \
+                          x, (const T*)a, a_mult, (const T*)a2, a2_mult, (const T*)wa, rows, (const T*)w, w_off, width, eps, (T*)out))
+    NVS_ROW_CASES(per, NVS_ROW)
+#undef NVS_ROW
+    return nvs_check_launch("nvs_sandwich_norm (rows in registers)");
+  }
   NVS_DISPATCH(dtype, sandwich_norm_kernel<T><<<dim3((unsigned)nrows), dim3(threads_for(width)), 0, (hipStream_t)stream>>>(
                           x, (const T*)a, a_mult, (const T*)a2, a2_mult, (const T*)wa, rows, (const T*)w, w_off, width, eps, sum, (T*)out));
   return nvs_check_launch("nvs_sandwich_norm");
@@ -468,6 +582,16 @@ extern "C" int nvs_embed_norm(const void* table, int dtype, const int64_t* ids, 
                               void* stream) {
   NVS_REQUIRE(table && ids && w && x && n >= 0 && width > 0, "nvs_embed_norm: bad argument (width %d)", width);
   if (n == 0) return NVS_OK;
+  int row_threads = 0;
+  const int per = row_plan(width, (uintptr_t)table | (uintptr_t)w | (uintptr_t)x, &row_threads);
+  if (per) {
+#define NVS_ROW(PER)                                                                                                        \
+  NVS_DISPATCH(dtype, embed_norm_row_kernel<T, PER><<<dim3((unsigned)n), dim3(row_threads), 0, (hipStream_t)stream>>>(        \
+                          (const T*)table, ids, width, (const T*)w, eps, x))
+    NVS_ROW_CASES(per, NVS_ROW)
+#undef NVS_ROW
+    return nvs_check_launch("nvs_embed_norm (rows in registers)");
+  }
   NVS_DISPATCH(dtype, embed_norm_kernel<T><<<dim3((unsigned)n), dim3(threads_for(width)), 0, (hipStream_t)stream>>>(
                           (const T*)table, ids, width, (const T*)w, eps, x));
   return nvs_check_launch("nvs_embed_norm");

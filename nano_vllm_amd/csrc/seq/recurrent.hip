@@ -604,30 +604,43 @@ __global__ void gated_group_norm_kernel(const float* __restrict__ y, const T* __
   }
 }
 
-// Norm first, then the gate, for groups of up to 256 entries: a wavefront per group, four wavefronts share a row's groups.
-template <typename T, int PER>
+// Norm first, then the gate, for groups of up to 256 entries: a wavefront per group; the four wavefronts of a workgroup take groups
+// blockIdx.y * 4 + wave, + 4 gridDim.y, ... of a row. A lane holds PER neighbouring entries (VEC: loaded and stored as one piece).
+template <typename T, int PER, bool VEC>
 __global__ __launch_bounds__(256) void norm_gate_rows_kernel(const float* __restrict__ y, const T* __restrict__ z, int64_t z_stride,
                                                              const T* __restrict__ w, int wlen, int inner, int groups, float eps, int silu,
                                                              const float* __restrict__ den, T* __restrict__ out) {
   const int64_t t = blockIdx.x;
-  const int gsz = inner / groups, lane = threadIdx.x & 63;
-  for (int g = threadIdx.x >> 6; g < groups; g += 4) {
+  const int gsz = inner / groups, lane = threadIdx.x & 63, c = lane * PER;
+  for (int g = blockIdx.y * 4 + (threadIdx.x >> 6); g < groups; g += 4 * gridDim.y) {
     const int c0 = g * gsz;
     const float dinv = den ? 1.f / den[t * groups + g] : 1.f;
-    float v[PER], gz[PER], ss = 0.f;
+    const T* wg = w + (wlen < inner ? 0 : c0);
+    float v[PER], gz[PER], wv[PER], ss = 0.f;
+    if (VEC) {
+      ldp<PER>(y + t * inner + c0 + c, v);
+      ldp<PER>(z + t * z_stride + c0 + c, gz);
+      ldp<PER>(wg + c, wv);
+    } else {
 #pragma unroll
-    for (int i = 0; i < PER; ++i) {
-      const int c = lane + 64 * i;
-      const bool in = c < gsz;
-      v[i] = in ? y[t * inner + c0 + c] * dinv : 0.f;
-      gz[i] = in ? ldf(z + t * z_stride + c0 + c) : 0.f;
-      ss += v[i] * v[i];
+      for (int i = 0; i < PER; ++i) {
+        const bool in = c + i < gsz;
+        v[i] = in ? y[t * inner + c0 + c + i] : 0.f;
+        gz[i] = in ? ldf(z + t * z_stride + c0 + c + i) : 0.f;
+        wv[i] = in ? ldf(wg + c + i) : 0.f;
+      }
     }
+#pragma unroll
+    for (int i = 0; i < PER; ++i) v[i] *= dinv, ss += v[i] * v[i];
     const float r = 1.f / sqrtf(wave_sum(ss) / (float)gsz + eps);
 #pragma unroll
-    for (int i = 0; i < PER; ++i) {
-      const int c = lane + 64 * i;
-      if (c < gsz) stf(out + t * inner + c0 + c, v[i] * r * ldf(w + (wlen < inner ? c : c0 + c)) * ((silu ? gz[i] : 1.f) / (1.f + expf(-gz[i]))));
+    for (int i = 0; i < PER; ++i) v[i] *= r * wv[i] * ((silu ? gz[i] : 1.f) / (1.f + expf(-gz[i])));
+    if (VEC) {
+      stp<PER>(out + t * inner + c0 + c, v);
+    } else {
+#pragma unroll
+      for (int i = 0; i < PER; ++i)
+        if (c + i < gsz) stf(out + t * inner + c0 + c + i, v[i]);
     }
   }
 }
@@ -879,12 +892,21 @@ extern "C" int nvs_gated_group_norm(const float* y, const void* z, int64_t z_str
   NVS_REQUIRE(n <= 65535ll * 65535ll, "nvs_gated_group_norm: step too large");
   const int gsz = inner / groups;
   if (order >= 1 && gsz <= 256 && groups >= 4) {
-#define NVS_NORM_GATE(PER)                                                                                                        \
-  NVS_DISPATCH(dtype, norm_gate_rows_kernel<T, PER><<<dim3((unsigned)n), dim3(256), 0, (hipStream_t)stream>>>(                      \
+    const int per = gsz <= 64 ? 1 : (gsz <= 128 ? 2 : 4);
+    const bool vec = gsz == 64 * per && z_stride % per == 0 && ((uintptr_t)y | (uintptr_t)z | (uintptr_t)w | (uintptr_t)out) % 16 == 0;
+    const dim3 grid((unsigned)n, n >= 4096 ? (unsigned)((groups + 15) / 16) : (unsigned)((groups + 3) / 4));
+#define NVS_NORM_GATE(PER, VEC)                                                                                                   \
+  NVS_DISPATCH(dtype, norm_gate_rows_kernel<T, PER, VEC><<<grid, dim3(256), 0, (hipStream_t)stream>>>(                              \
                           y, (const T*)z, z_stride, (const T*)w, wlen, inner, groups, eps, order == 2, den, (T*)out))
-    if (gsz <= 64) NVS_NORM_GATE(1);
-    else if (gsz <= 128) NVS_NORM_GATE(2);
-    else NVS_NORM_GATE(4);
+    if (vec) {
+      if (per == 1) NVS_NORM_GATE(1, true);
+      else if (per == 2) NVS_NORM_GATE(2, true);
+      else NVS_NORM_GATE(4, true);
+    } else {
+      if (per == 1) NVS_NORM_GATE(1, false);
+      else if (per == 2) NVS_NORM_GATE(2, false);
+      else NVS_NORM_GATE(4, false);
+    }
 #undef NVS_NORM_GATE
     return nvs_check_launch("nvs_gated_group_norm (rows)");
   }

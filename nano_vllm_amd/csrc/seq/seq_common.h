@@ -70,6 +70,23 @@ __device__ __forceinline__ void stv(bf16_t* p, const float (&v)[VEC]) {
   }
 }
 
+// N (1, 2 or 4) consecutive elements in one piece (the address is aligned to the piece)
+template <int N, typename T>
+__device__ __forceinline__ void ldp(const T* p, float (&v)[N]) {
+  typedef __attribute__((ext_vector_type(N))) T vec_t;
+  const vec_t f = *(const vec_t*)p;
+#pragma unroll
+  for (int i = 0; i < N; ++i) v[i] = (float)f[i];
+}
+template <int N, typename T>
+__device__ __forceinline__ void stp(T* p, const float (&v)[N]) {
+  typedef __attribute__((ext_vector_type(N))) T vec_t;
+  vec_t f;
+#pragma unroll
+  for (int i = 0; i < N; ++i) f[i] = (T)v[i];
+  *(vec_t*)p = f;
+}
+
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll
   for (int o = 32; o > 0; o >>= 1) v += __shfl_xor(v, o, 64);

@@ -128,17 +128,57 @@ def test_embedding_norm_gated_lookup_and_rounded_sums(dtype, tol):
 
 
 @pytest.mark.parametrize("dtype,tol", BOTH)
+@pytest.mark.parametrize("W", [4, 260, 1028, 4096, 5000, 8192, 9000])
+def test_row_norms_of_wide_rows(dtype, tol, W):
+    """Rows that fit a workgroup's registers (one to eight accesses per thread) and one that does not: the norm ahead of a feed-forward,
+    the normed embedding, and the last norm on selected rows with a branch that is normed and added only there."""
+    from nano_vllm_amd import ops_seq
+    g = torch.Generator().manual_seed(W)
+    n = 5
+    x, a, w, wa = torch.randn(n, W, generator=g), bf(torch.randn(n, W, generator=g)), bf(1 + 0.2 * torch.randn(W, generator=g)), bf(torch.randn(W, generator=g))
+    f = plain.f64
+    xd, out = dev(x), torch.empty(n, W, dtype=dtype, device="cuda")
+    ops_seq.add_group_norm(xd, dev(w, dtype), 1, EPS, out, dev(a, dtype))
+    close(xd, f(x) + f(a), 3e-6)
+    close(out, plain.norm(f(x) + f(a), f(w), EPS), tol)
+    rows = torch.tensor([3, 0, 3], dtype=torch.int32, device="cuda")
+    picked, xd = torch.empty(3, W, dtype=dtype, device="cuda"), dev(x)
+    ops_seq.offset_norm_rows(xd, rows, 3, dev(w, dtype), EPS, picked, w_off=0.0, a=dev(a, dtype), wa=dev(wa, dtype))
+    close(picked, plain.norm(f(x) + plain.norm(f(a), f(wa), EPS), f(w), EPS)[[3, 0, 3]], tol)
+    assert torch.equal(xd.cpu(), x), "selected rows are only read"
+    ids, emb = torch.tensor([2, 0, 2, 4]), torch.empty(4, W, device="cuda")
+    ops_seq.embed_norm(dev(a, dtype), dev(ids), dev(w, dtype), EPS, emb)
+    close(emb, plain.norm(f(a)[ids.numpy()], f(w), EPS), 3e-6)
+
+
+@pytest.mark.parametrize("dtype,tol", BOTH)
+@pytest.mark.parametrize("groups,gsz,n", [(4, 64, 5), (6, 128, 70), (5, 256, 3), (7, 20, 9), (4, 130, 4200), (3, 32, 6), (40, 128, 4100)])
+@pytest.mark.parametrize("silu", [False, True])
+def test_norm_per_head_then_gate(dtype, tol, groups, gsz, n, silu):
+    from nano_vllm_amd import ops_seq
+    g = torch.Generator().manual_seed(groups * gsz)
+    inner = groups * gsz
+    y, z, w = torch.randn(n, inner, generator=g), bf(torch.randn(n, inner + 5, generator=g)), bf(1 + 0.2 * torch.randn(gsz, generator=g))
+    out = torch.empty(n, inner, dtype=dtype, device="cuda")
+    ops_seq.gated_group_norm(dev(y), dev(z, dtype)[:, 5:], dev(w, dtype), groups, EPS, out, norm_first=True, silu=silu)
+    zf = plain.f64(z)[:, 5:]
+    want = plain.norm(plain.f64(y).reshape(n, groups, gsz), plain.f64(w), EPS).reshape(n, inner) * (plain.silu(zf) if silu else plain.sigmoid(zf))
+    close(out, want, tol if dtype == torch.bfloat16 else 1e-5)
+
+
+@pytest.mark.parametrize("dtype,tol", BOTH)
 @pytest.mark.parametrize("taps,C", [(1, 7), (2, 40), (3, 300), (4, 64), (6, 20)])
 def test_convolution_of_short_and_long_portions(dtype, tol, taps, C):
-    """Steps of short portions walk the taps in registers, others take a thread per token: both continue from the same state."""
+    """Steps of short portions walk the taps in registers, long steps take tiles of tokens, others a thread per token: all continue
+    from the same state."""
     from nano_vllm_amd import ops_seq
     g = torch.Generator().manual_seed(taps)
-    T = 40
-    u, w = bf(torch.randn(T, C + 2, generator=g)), bf(torch.randn(C, taps, generator=g))
+    T = 640
+    u, w = bf(torch.randn(T, C + 4, generator=g)), bf(torch.randn(C, taps, generator=g))
     want = plain.short_conv(plain.f64(u)[:, :C], plain.f64(w))
     state = torch.full((3, taps - 1, C), 5.0, device="cuda")
     at, rows = 0, []
-    for c in (1, 1, 2, 9, 1, 3, 20, 1, 1, 1):
+    for c in (1, 1, 2, 9, 1, 3, 20, 1, 1, 1, 300, 2, 298):
         out = torch.empty(c, C, dtype=dtype, device="cuda")
         ops_seq.causal_conv(dev(u[at:at + c], dtype)[:, :C], dev(w, dtype), None, 1, portions([c], [at], [1]), state, out)
         rows.append(out)
