@@ -285,7 +285,10 @@ CUTS = [[0], [97, 2, 1, 1, 30, 2, 1, 1, 1, 44], [1] * 40 + [2] * 20 + [100]]
     (1, 1, 40, 40, 33, 50, 16, 16, 12.0),     # blocks longer than the window and than a page
     (6, 2, 136, 72, 16, 8, 64, 40, 20.0),     # long heads
     (2, 2, 16, 200, 500, 4, 48, 16, 9.0),     # a window that nothing leaves
-    (20, 2, 8, 8, 50, 2, 64, 8, 6.0)])
+    (20, 2, 8, 8, 50, 2, 64, 8, 6.0),
+    # every size of the matrix-core kernels
+    (4, 1, 72, 40, 20, 3, 16, 8, 7.0), (2, 2, 128, 128, 30, 6, 32, 64, 20.0), (4, 4, 104, 144, 25, 4, 16, 8, 9.0),
+    (2, 1, 192, 64, 18, 5, 16, 16, 11.0), (3, 1, 160, 160, 22, 7, 64, 32, 8.0), (2, 1, 256, 256, 26, 9, 32, 128, 15.0)])
 def test_window_with_pooled_blocks_against_the_plain_loop(H, G, d, dv, size, pool, block, rot_dims, cap, dtype, path, tol):
     T = 180
     m, w, h = attention_case(H, G, d, dv, size, pool, rot_dims, cap, T, seed=H * 100 + d)
