@@ -21,7 +21,9 @@ LIBDIR = os.environ.get("NVL_LIBDIR") or os.path.join(HERE, "lib")   # (NVL_LIBD
 LIB = os.path.join(LIBDIR, "libnvl_hip.so")
 STAMP = os.path.join(LIBDIR, "libnvl_hip.stamp")
 ARCH = "gfx950"
-FLAGS = ["-O3", "-std=c++17", "-fPIC", "-Wall", "-Wno-unused-function", "-fno-gpu-rdc"]
+# packed 32-bit float instructions are kept out of every kernel: the compiler makes them from ordinary float code by itself, and some
+# of their forms have given wrong results on this hardware
+FLAGS = ["-O3", "-std=c++17", "-fPIC", "-Wall", "-Wno-unused-function", "-fno-gpu-rdc", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
 if os.environ.get("NVL_PROBES") == "1":       # probe build: the kernels' measurement switches (NVL_WIDE_DBG / _DEBUG) exist
     FLAGS.append("-DNVL_PROBES")
     FLAGS += os.environ.get("NVL_PROBE_FLAGS", "").split()      # e.g. -DNVL_PF_PACKED: a compile-time variant under A/B
@@ -120,8 +122,7 @@ def build(force: bool = False, verbose: bool = False) -> str:
 # ---- libnvl_seq.so ------------------------------------------------------------------------------------------------
 SEQ_CSRC = os.path.join(CSRC, "seq")
 LIB_SEQ = os.path.join(LIBDIR, "libnvl_seq.so")
-# packed 32-bit float instructions are kept out of these kernels: their recurrences and norms are 32-bit throughout
-SEQ_FLAGS = FLAGS + ["-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops"]
+SEQ_FLAGS = FLAGS
 
 
 def seq_sources() -> list[str]:
