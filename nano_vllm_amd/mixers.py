@@ -422,8 +422,8 @@ class DeltaMixer(nn.Module):
     q and k become unit vectors per head, q times dim^(-1/2); with a step size beta = sigmoid(W_b h) and a decay g per head,
         S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q          (state and everything on this line in 32-bit),
     g = exp(-exp(A_log) softplus(W_a h + dt_bias)) — or, with decay_rank > 0, one per head and KEY CHANNEL, from W_a2 (W_a1 h).
-    Every head's o is divided by its root mean square, times `norm` (one set of vdim weights), times silu(W_g h) — or, with
-    gate_rank > 0, sigmoid(W_g2 (W_g1 h)) — and projected. ONE in-projection [q | k | v | g or g1 | a or a1 | b]."""
+    The read-out is RMS-normed head by head (`norm`: one set of vdim weights for all of them), gated by silu(W_g h) — or, with
+    gate_rank > 0, by sigmoid(W_g2 (W_g1 h)) — and projected. ONE in-projection [q | k | v | g or g1 | a or a1 | b]."""
 
     def __init__(self, width: int, heads: int, kv_heads: int, dim: int, vdim: int, taps: int, eps: float, decay_rank: int = 0, gate_rank: int = 0):
         super().__init__()
