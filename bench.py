@@ -29,9 +29,9 @@ driver's fields it carries
                  race keys with the draws replayed (a by-product of the cpu_baseline leg: the timed
                  oracle pass is teacher-forced with the engine's tokens).
 
-`python bench.py --compare-families [--families ligidra,lobidra,pefazen,nokipel,foduzen,qwen3] [--sizes 1k,4k]` is a different measurement with a
-line of its own (metric "family_compare"): prefill and decode throughput of the Ligidra, Lobidra, Pefazen, Nokipel and Foduzen families at layer
-sizes of real models beside Qwen3 at equal width and depth. The default command above is unchanged by it.
+`python bench.py --compare-families [--families reselorn,ligidra,lobidra,pefazen,nokipel,foduzen,qwen3] [--sizes 1k,4k]` is a different measurement with a
+line of its own (metric "family_compare"): prefill and decode throughput of the Reselorn, Ligidra, Lobidra, Pefazen, Nokipel and Foduzen
+families at layer sizes of real models beside Qwen3 at equal width and depth. The default command above is unchanged by it.
 """
 from __future__ import annotations
 
@@ -89,9 +89,9 @@ def parse():
     ap.add_argument("--kv-cache-dtype", default="bf16", choices=["bf16", "fp8"],
                     help="fp8: opt-in OCP e4m3 KV cache (outside the reference's numerics; never the headline)")
     ap.add_argument("--compare-families", action="store_true",
-                    help="instead of the headline workload: prefill and decode throughput of the Ligidra, Lobidra, Pefazen, Nokipel and Foduzen families at "
-                         "layer sizes of real models (random weights) beside Qwen3 models of equal width / depth, one JSON line")
-    ap.add_argument("--families", default="ligidra,lobidra,pefazen,nokipel,foduzen,qwen3", help="with --compare-families: which of the six to run")
+                    help="instead of the headline workload: prefill and decode throughput of the Reselorn, Ligidra, Lobidra, Pefazen, Nokipel and Foduzen "
+                         "families at layer sizes of real models (random weights) beside Qwen3 models of equal width / depth, one JSON line")
+    ap.add_argument("--families", default="reselorn,ligidra,lobidra,pefazen,nokipel,foduzen,qwen3", help="with --compare-families: which of the seven to run")
     ap.add_argument("--sizes", default="1k,4k", help="with --compare-families: layer sizes to run (1k, 4k)")
     return ap.parse_args()
 
@@ -190,6 +190,17 @@ def ligidra_config(width: int, ff: int, heads: int, kv_heads: int, layers: int, 
     return {"architecture": "Ligidra", "layers": out, "norm": {"eps": 1e-6}, "token_side": {"dim": width // 16}, "vocab": vocab, "width": width}
 
 
+def reselorn_config(width: int, ff: int, heads: int, kv_heads: int, layers: int, vocab: int) -> dict:
+    """Layers of a real model's size: 128-wide heads with a window of 1,024 positions, half of every head rotated with scaled frequencies,
+    values mixed with the first layer's; every second layer has 32 experts of a quarter of the dense width (4 per token) plus a
+    shared one, the others (from the first on) a dense feed-forward."""
+    mixer = {"heads": heads, "kv_heads": kv_heads, "dim": 128, "vdim": 128, "scale": 128 ** -0.5, "mask": {"size": 1024}, "v_mix": True,
+             "rot": {"dims": 64, "base": 500000.0, "scaling": {"factor": 4.0, "fast": 32.0, "slow": 1.0, "original": 4096}}}
+    moe = {"kind": "moe", "expert": {"ff": ff // 4}, "shared": {"ff": ff // 4}, "router": {"experts": 32, "top": 4}}
+    out = [{"type": "attention", "mixer": mixer, "mlp": moe if i % 2 else {"kind": "dense", "ff": ff}} for i in range(layers)]
+    return {"architecture": "Reselorn", "layers": out, "norm": {"eps": 1e-6}, "vocab": vocab, "width": width}
+
+
 FAMILY_SIZES = {   # name: (width, ff, heads, kv heads, layers, the Qwen3 shape of the same width / depth)
     "1k": (1024, 3072, 16, 8, 4, "qwen3-0.6b-4l"),
     "4k": (4096, 12288, 32, 8, 2, "qwen3-8b-2l"),
@@ -211,9 +222,9 @@ def compare_families(args) -> dict:
         width, ff, heads, kv, layers, qname = FAMILY_SIZES[size]
         for family in args.families.split(","):
             path = os.path.join(tempfile.gettempdir(), f"nvl_cmp_{family}_{size}")
-            if family in ("foduzen", "nokipel", "pefazen", "lobidra", "ligidra"):
+            if family in ("foduzen", "nokipel", "pefazen", "lobidra", "ligidra", "reselorn"):
                 raw = {"foduzen": foduzen_config, "nokipel": nokipel_config, "pefazen": pefazen_config,
-                       "lobidra": lobidra_config, "ligidra": ligidra_config}[family](width, ff, heads, kv, layers, vocab)
+                       "lobidra": lobidra_config, "ligidra": ligidra_config, "reselorn": reselorn_config}[family](width, ff, heads, kv, layers, vocab)
                 os.makedirs(path, exist_ok=True)
                 with open(os.path.join(path, "config.json"), "w") as fh:
                     json.dump(raw, fh)

@@ -56,6 +56,13 @@ int nvs_add_group_norm(float* x, const void* a, float a_mult, const float* b, co
 int nvs_sandwich_norm(float* x, const void* a, float a_mult, const void* a2, float a2_mult, const void* wa, const int32_t* rows,
                       int64_t nrows, const void* w, float w_off, int dtype, int width, float eps, float* sum, void* out, void* stream);
 
+/* Residual update of a sublayer whose output is normed, with a layer scale, and the next sublayer's input. The output is
+ * y[t, :] = a[t, :] (nullable) + sum_k wts[t, k] * rows[pair_row[t, k], :] (top choices of a routed layer, see nvs_moe_combine; top 0: none;
+ * pair_row < 0: skipped); x[t, :] += rms(y[t, :]) * w * ls (ls nullable: no scale); out (nullable) receives the new x in `dtype`. a, rows (row
+ * stride ldr), w, ls in `dtype`; sums in 32-bit. width <= 16384. */
+int nvs_branch_norm(float* x, const void* a, const void* rows, int64_t ldr, const int32_t* pair_row, const float* wts, int top, int dtype,
+                    int64_t n, const void* w, const void* ls, int width, float eps, void* out, void* stream);
+
 /* x[t, :] = rms(table[ids[t], :]) * w, 32-bit. */
 int nvs_embed_norm(const void* table, int dtype, const int64_t* ids, int64_t n, int width, const void* w, float eps, float* x, void* stream);
 
@@ -173,6 +180,17 @@ void nvs_delta_force(int mode);
 int nvs_knorm_kvstore(const void* k, const void* v, int64_t stride, int dtype, const void* knorm, float eps, int G, int d, int dv,
                       int block_size, const int32_t* slots, const int64_t* pos, const float* rot_freq, int rot_dims, int64_t n,
                       void* k_cache, void* v_cache, void* stream);
+
+/* Everything between a fused projection and nvs_window_attn for heads that are normed AFTER their rotation. q [n, H, d], k [n, G, d] and
+ * v [n, G, dv] are column ranges of one projection output (row stride `stride`, `dtype`). Per query and key head: the leading rot_dims
+ * entries turn by pos[t] * rot_freq[i] (32-bit), i < rot_dims / 2, in pairs (2i, 2i+1) or, with rot_halves, (i, i + rot_dims / 2), cos and sin
+ * multiplied by rot_mag; with `unit` the head is then divided by sqrt(mean over d of its squares + eps). Queries are also multiplied by
+ * q_scale and written back IN PLACE; keys go to the cache as nvs_knorm_kvstore's do (slots[t] < 0: not stored). Values: with v0 (nullable,
+ * row stride v0_stride) v <- (1 - *mix) v + *mix v0 (mix: one 32-bit number on the device), then the paged store. d, dv <= 1024. */
+int nvs_qkv_store(void* q, const void* k, const void* v, int64_t stride, int dtype, int H, int G, int d, int dv, const int64_t* pos,
+                  const float* rot_freq, int rot_dims, int rot_halves, float rot_mag, int unit, float eps, float q_scale, const void* v0,
+                  int64_t v0_stride, const float* mix, int block_size, const int32_t* slots, int64_t n, void* k_cache, void* v_cache,
+                  void* stream);
 
 /* Locally masked softmax attention over the paged cache, one query per token row, any d, dv <= 1024.
  * q [n, H, d] (row stride q_stride), RMS-normed per head with qnorm [d] here (NULL: none), then rotated like the keys

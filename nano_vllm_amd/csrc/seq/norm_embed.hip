@@ -20,7 +20,7 @@ int nvs_check_launch(const char* what) {
   }
   return NVS_OK;
 }
-extern "C" int nvs_abi_version(void) { return 6; }   // 6: token-shift norms, gated lookups, the gated delta rule, pooled blocks behind an attention window, capped scores
+extern "C" int nvs_abi_version(void) { return 7; }   // 7: rotated and normed queries / keys with blended values in one store, norms on a sublayer's output with a layer scale
 extern "C" const char* nvs_last_error(void) { return g_err; }
 
 namespace {
@@ -317,6 +317,87 @@ __global__ __launch_bounds__(256) void sandwich_row_kernel(float* __restrict__ x
   }
 }
 
+// A sublayer whose OUTPUT is normed, with a layer scale: y[t] = a[t] + sum_k wts[t, k] rows[pair_row[t, k]] (either part may be absent: the
+// output of a product, or a token's chosen experts beside a shared one), x[t] += rms(y[t]) * w * ls, and the new row once more in the
+// activation type for the next sublayer's products. One workgroup per row, y and x in registers (PER accesses of four columns per thread).
+template <typename T, int PER>
+__global__ __launch_bounds__(256) void branch_norm_row_kernel(float* __restrict__ x, const T* __restrict__ a, const T* __restrict__ rows, int64_t ldr,
+                                                              const int32_t* __restrict__ pair_row, const float* __restrict__ wts, int top,
+                                                              const T* __restrict__ w, const T* __restrict__ ls, int width, float eps,
+                                                              T* __restrict__ out) {
+  __shared__ float red[16];
+  const int64_t t = blockIdx.x;
+  float v[PER][4], y[PER][4];
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int c = (i * blockDim.x + threadIdx.x) * 4;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) y[i][e] = 0.f;
+    if (c >= width) continue;
+    ldv<4>(x + t * width + c, v[i]);
+    if (a) ldv<4>(a + t * width + c, y[i]);
+  }
+  for (int k = 0; k < top; ++k) {
+    const int r = pair_row[t * top + k];
+    if (r < 0) continue;                            // (uniform over the workgroup)
+    const float p = wts[t * top + k];
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+      const int c = (i * blockDim.x + threadIdx.x) * 4;
+      if (c >= width) continue;
+      float u[4];
+      ldv<4>(rows + (int64_t)r * ldr + c, u);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) y[i][e] += p * u[e];
+    }
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < PER; ++i)
+#pragma unroll
+    for (int e = 0; e < 4; ++e) ss += y[i][e] * y[i][e];
+  const float k = 1.f / sqrtf(block_sum(ss, red) / (float)width + eps);
+#pragma unroll
+  for (int i = 0; i < PER; ++i) {
+    const int c = (i * blockDim.x + threadIdx.x) * 4;
+    if (c >= width) continue;
+    float g[4], s[4] = {1.f, 1.f, 1.f, 1.f};
+    ldv<4>(w + c, g);
+    if (ls) ldv<4>(ls + c, s);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[i][e] += y[i][e] * k * g[e] * s[e];
+    stv<4>(x + t * width + c, v[i]);
+    if (out) stv<4>(out + t * width + c, v[i]);
+  }
+}
+
+// the same for any width: y in LDS (every thread only touches its own columns)
+template <typename T>
+__global__ __launch_bounds__(256) void branch_norm_kernel(float* __restrict__ x, const T* __restrict__ a, const T* __restrict__ rows, int64_t ldr,
+                                                          const int32_t* __restrict__ pair_row, const float* __restrict__ wts, int top,
+                                                          const T* __restrict__ w, const T* __restrict__ ls, int width, float eps,
+                                                          T* __restrict__ out) {
+  extern __shared__ __attribute__((aligned(16))) float branch_lds[];
+  __shared__ float red[16];
+  const int64_t t = blockIdx.x;
+  float ss = 0.f;
+  for (int c = threadIdx.x; c < width; c += blockDim.x) {
+    float y = a ? ldf(a + t * width + c) : 0.f;
+    for (int k = 0; k < top; ++k) {
+      const int r = pair_row[t * top + k];
+      if (r >= 0) y += wts[t * top + k] * ldf(rows + (int64_t)r * ldr + c);
+    }
+    branch_lds[c] = y;
+    ss += y * y;
+  }
+  const float k = 1.f / sqrtf(block_sum(ss, red) / (float)width + eps);
+  for (int c = threadIdx.x; c < width; c += blockDim.x) {
+    const float v = x[t * width + c] + branch_lds[c] * k * ldf(w + c) * (ls ? ldf(ls + c) : 1.f);
+    x[t * width + c] = v;
+    if (out) stf(out + t * width + c, v);
+  }
+}
+
 // x[t] = rms(table[ids[t]]) * w: one workgroup per token, the row in registers (PER accesses of four columns per thread)
 template <typename T, int PER>
 __global__ __launch_bounds__(256) void embed_norm_row_kernel(const T* __restrict__ table, const int64_t* __restrict__ ids, int width,
@@ -567,6 +648,31 @@ extern "C" int nvs_sandwich_norm(float* x, const void* a, float a_mult, const vo
   NVS_DISPATCH(dtype, sandwich_norm_kernel<T><<<dim3((unsigned)nrows), dim3(threads_for(width)), 0, (hipStream_t)stream>>>(
                           x, (const T*)a, a_mult, (const T*)a2, a2_mult, (const T*)wa, rows, (const T*)w, w_off, width, eps, sum, (T*)out));
   return nvs_check_launch("nvs_sandwich_norm");
+}
+
+extern "C" int nvs_branch_norm(float* x, const void* a, const void* rows, int64_t ldr, const int32_t* pair_row, const float* wts, int top, int dtype,
+                               int64_t n, const void* w, const void* ls, int width, float eps, void* out, void* stream) {
+  NVS_REQUIRE(x && w && n >= 0 && width > 0 && width <= 16384 && top >= 0 && (a || top > 0), "nvs_branch_norm: bad argument (width %d, %d choices)", width, top);
+  NVS_REQUIRE(top == 0 || (rows && pair_row && wts && ldr >= width), "nvs_branch_norm: %d choices without their rows", top);
+  if (n == 0) return NVS_OK;
+  int row_threads = 0;
+  const uintptr_t al = (uintptr_t)x | (uintptr_t)a | (uintptr_t)(top ? rows : nullptr) | (uintptr_t)w | (uintptr_t)ls | (uintptr_t)out;
+  const int per = top == 0 || ldr % 4 == 0 ? row_plan(width, al, &row_threads) : 0;
+  if (per) {
+#define NVS_ROW(PER)                                                                                                             \
+  NVS_DISPATCH(dtype, branch_norm_row_kernel<T, PER><<<dim3((unsigned)n), dim3(row_threads), 0, (hipStream_t)stream>>>(            \
+                          x, (const T*)a, (const T*)rows, ldr, pair_row, wts, top, (const T*)w, (const T*)ls, width, eps, (T*)out))
+    NVS_ROW_CASES(per, NVS_ROW)
+#undef NVS_ROW
+    return nvs_check_launch("nvs_branch_norm (rows in registers)");
+  }
+  const size_t lds = (size_t)width * sizeof(float);      // (at most 64 KB)
+  NVS_DISPATCH(dtype, {
+    if (lds > 48 * 1024) (void)hipFuncSetAttribute((const void*)branch_norm_kernel<T>, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    branch_norm_kernel<T><<<dim3((unsigned)n), dim3(threads_for(width)), lds, (hipStream_t)stream>>>(
+        x, (const T*)a, (const T*)rows, ldr, pair_row, wts, top, (const T*)w, (const T*)ls, width, eps, (T*)out);
+  });
+  return nvs_check_launch("nvs_branch_norm");
 }
 
 extern "C" int nvs_scale_softcap(const void* in, int dtype, float scale, float cap, int64_t numel, float* out, void* stream) {

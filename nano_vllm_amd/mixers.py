@@ -3,7 +3,8 @@
   WindowAttention     paged softmax attention with a local mask (a sliding window, or blocks of positions, or none), any
                       query / value head size, optional per-head q/k RMS norm, optional rotation of the leading dimensions
                       in interleaved pairs, optional sigmoid output gate, capped scores, a norm over the whole query / key
-                      projection, means over blocks of positions behind the window, another layer's keys and values
+                      projection, means over blocks of positions behind the window, another layer's keys and values; heads normed
+                      after a rotation in either pairing, values blended with an earlier layer's
   AttentionMixer      fused q | k | v projection (biased or not) -> WindowAttention -> out projection
   ConvAttentionMixer  attention whose query and key projections pass a short stateful causal convolution, whose keys (before
                       rotation) are also its values, with a constant or learned sink in the softmax and a gate per head
@@ -29,9 +30,12 @@
   XIELUFeedForward    up -> xIELU -> down
   ClampedGLU          [gate | up] -> min(g, limit) sigmoid(alpha g) (clamp(u) + 1) -> down
   GeluFeedForward     up -> GELU (tanh form) -> down
+  SiluGLU             [gate | up] -> silu(g) u -> down
+  BranchNorm          norm on a sublayer's OUTPUT with a layer scale: the residual add and the next sublayer's input in one kernel,
+                      for a routed layer the weighted sum of a token's experts too
   RoutedExperts       mixture of experts (gated SiLU units, or ungated squared-ReLU units): softmax or sigmoid router with a
                       choice-only correction, choice limited to the best groups of experts, weights renormalised or not,
-                      pass-through experts, optional shared expert with a sigmoid gate per token; or, instead of a router, a
+                      pass-through experts, biased logits, optional shared expert with a sigmoid gate per token; or, instead of a router, a
                       table from token ids to experts with equal weights
 
 Every constant a design may change is a constructor argument. Matrix products are the vendor library's (F.linear /
@@ -53,7 +57,7 @@ from .attn_meta import get_context
 
 
 def _param(*shape, dtype=None):
-    return nn.Parameter(torch.zeros(*shape, dtype=dtype), requires_grad=False)
+    return nn.Parameter(torch.zeros(shape, dtype=dtype), requires_grad=False)
 
 
 def _copy_into(dst: torch.Tensor):
@@ -69,8 +73,12 @@ class WindowAttention(nn.Module):
     def __init__(self, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, window: int, eps: float,
                  qk_norm: bool = True, block_size: int = 256, chunk: int = 0, rot_dims: int = 0, rot_base: float = 10000.0,
                  rot_freqs: list | None = None, sink: str | None = None, q_temp: tuple | None = None, gate_per_head: bool = False,
-                 norm_rows: bool = False, softcap: float = 0.0, pool: int = 0, source: "WindowAttention | None" = None):
-        """norm_rows: the query and key norms are over the whole projection (all heads together), not per head. softcap > 0: scores
+                 norm_rows: bool = False, softcap: float = 0.0, pool: int = 0, source: "WindowAttention | None" = None,
+                 rot_halves: bool = False, rot_mag: float = 1.0, qk_unit: bool = False, v_mix: bool = False):
+        """qk_unit: query and key heads are divided by their root mean square (no weights) AFTER their rotation. rot_halves: the pairs that
+        turn are (i, i + rot_dims / 2). rot_mag: factor on cos and sin. v_mix: forward() may be handed the values of an earlier layer
+        (`first`), v becomes (1 - vmix) v + vmix first with the learned number `vmix`. Any of these takes everything between
+        the projection and the attention call into one kernel (ops_seq.qkv_store). norm_rows: the query and key norms are over the whole projection (all heads together), not per head. softcap > 0: scores
         become softcap tanh(score / softcap). pool > 0 (behind a window): beside the window's tokens a query sees the mean key and
         value of every block of `pool` positions that lies wholly before it. source: an earlier layer's attention whose cached
         keys and values this one reads instead of keeping its own (its k and v are then None).
@@ -101,6 +109,10 @@ class WindowAttention(nn.Module):
         # frequencies in double precision on the host, rounded once; angles are position * frequency in 32-bit
         freqs = rot_freqs if rot_freqs is not None else [float(rot_base) ** (-2.0 * i / rot_dims) for i in range(rot_dims // 2)]
         self.register_buffer("rot_freq", torch.tensor(freqs, dtype=torch.float32) if rot_dims else None, persistent=False)
+        self.stored_ready = bool(qk_unit or rot_halves or rot_mag != 1.0 or v_mix)      # queries and keys are finished by the store kernel
+        assert not self.stored_ready or not (qk_norm or norm_rows or pool or source is not None), "not with weighted norms, pooled blocks or a borrowed cache"
+        self.rot_halves, self.rot_mag, self.qk_unit = bool(rot_halves), float(rot_mag), bool(qk_unit)
+        self.vmix = _param(dtype=torch.float32) if v_mix else None
         self.q_norm = _param(heads * dim if norm_rows else dim) if qk_norm else None
         self.k_norm = _param(kv_heads * dim if norm_rows else dim) if qk_norm and source is None else None
         self.k_cache = self.v_cache = None            # [pages * block_size, G, d] / [..., G, dv] (values page-transposed), from the runner
@@ -131,8 +143,17 @@ class WindowAttention(nn.Module):
         rows = ops_seq.pool_rows(self.block_size, self.pool)
         return {"pool_k": (rows, self.G, self.d), "pool_v": (rows // 8, self.G, self.dv, 8)}
 
-    def forward(self, q, k, v, gate, positions: torch.Tensor | None = None) -> torch.Tensor:
+    def forward(self, q, k, v, gate, positions: torch.Tensor | None = None, first: torch.Tensor | None = None) -> torch.Tensor:
         ctx = get_context()
+        if self.stored_ready:
+            rot = ops_seq.Rotation(self.rot_freq, self.rot_halves, self.rot_mag) if self.rot_freq is not None else None
+            ops_seq.qkv_store(q, k, v, self.H, self.G, self.d, self.dv, self.block_size, ctx.slot_mapping, self.k_cache, self.v_cache, positions,
+                              rot, self.qk_unit, self.eps, self.scale, first, self.vmix)
+            out = torch.empty(q.shape[0], self.H * self.dv, dtype=q.dtype, device=q.device)
+            ops_seq.window_attn(q, None, self.eps, gate, self.k_cache, self.v_cache, ctx.block_tables, self.block_size, ctx.portions, self.H, self.G,
+                                self.d, self.dv, 1.0, self.window, out, self.chunk, gate_per_head=self.gate_per_head, sink=self.sink,
+                                q_temp=self.q_temp, softcap=self.softcap)
+            return out
         own, q_row = self.owner, None
         means = self if self._own_pool else own
         if self.norm_rows:
@@ -180,13 +201,20 @@ class AttentionMixer(nn.Module):
                 out[name] = _copy_into(w)
         if isinstance(self.attn.sink, nn.Parameter):
             out["sink"] = _copy_into(self.attn.sink)
+        if self.attn.vmix is not None:
+            out["vmix"] = _copy_into(self.attn.vmix)
         return out
 
-    def forward(self, xh: torch.Tensor, positions: torch.Tensor) -> torch.Tensor:
+    def forward(self, xh: torch.Tensor, positions: torch.Tensor, values: list | None = None) -> torch.Tensor:
+        """values (with v_mix): a list that lives for one step; the first layer that gets it leaves its own values there (and uses them as
+        they are), every later one blends them into its own."""
         proj = F.linear(xh, self.in_w, self.in_b)
         q, k, _ = self.cols
         kv = (proj[:, q:q + k], proj[:, q + k:]) if k else (None, None)
-        return F.linear(self.attn(proj[:, :q], *kv, None, positions), self.o_w)
+        first = values[0] if values else None
+        if values is not None and not values:
+            values.append(kv[1])
+        return F.linear(self.attn(proj[:, :q], *kv, None, positions, first), self.o_w)
 
 
 def rotary_frequencies(dims: int, base: float, scaling: dict | None = None) -> tuple[list[float], float]:
@@ -711,6 +739,39 @@ class GeluFeedForward(nn.Module):
         return F.linear(act, self.down)
 
 
+class SiluGLU(nn.Module):
+    """W_down (silu(W_gate h) * W_up h)."""
+
+    def __init__(self, width: int, ff: int):
+        super().__init__()
+        self.ff, self.gu, self.down = ff, _param(2 * ff, width), _param(width, ff)
+
+    def named_loaders(self) -> dict:
+        return {"gate": _copy_into(self.gu[:self.ff]), "up": _copy_into(self.gu[self.ff:]), "down": _copy_into(self.down)}
+
+    def forward(self, xh: torch.Tensor) -> torch.Tensor:
+        act = torch.empty(xh.shape[0], self.ff, dtype=xh.dtype, device=xh.device)
+        ops_seq.glu_act(F.linear(xh, self.gu), self.ff, act, kind=0)
+        return F.linear(act, self.down)
+
+
+class BranchNorm(nn.Module):
+    """x += rms(y) * w * scale for a sublayer's output y (`scale`: one factor per channel), in place on the 32-bit residual, and the new
+    residual in the activation type. y may be a routed layer's parts (RoutedExperts.parts): they are summed on the way."""
+
+    def __init__(self, width: int, eps: float):
+        super().__init__()
+        self.eps, self.w, self.scale = eps, _param(width), _param(width)
+
+    def forward(self, x: torch.Tensor, y, out: torch.Tensor | None) -> None:
+        if isinstance(y, tuple):
+            rows, plan, wts, shared, gate = y
+            assert gate is None
+            ops_seq.branch_norm(x, shared, self.w, self.scale, self.eps, out, (rows, plan, wts))
+        else:
+            ops_seq.branch_norm(x, y, self.w, self.scale, self.eps, out)
+
+
 class ClampedGLU(nn.Module):
     """g = min(W_gate h, limit), u = clamp(W_up h, -limit, limit); W_down (g sigmoid(alpha g) (u + 1))."""
 
@@ -739,12 +800,12 @@ class RoutedExperts(nn.Module):
 
     def __init__(self, width: int, experts: int, ff: int, top: int, scale: float = 1.0, identity: int = 0, group_count: int = 1,
                  group_keep: int = 1, shared_ff: int = 0, gated: bool = True, sigmoid: bool = False, renorm: bool = True,
-                 table_vocab: int = 0, shared_gate: bool = True, corrected: bool = True):
+                 table_vocab: int = 0, shared_gate: bool = True, corrected: bool = True, router_bias: bool = False):
         """gated False: an expert is W_down max(W_up h, 0)^2 (checkpoint names e<i>.up / e<i>.down). sigmoid: scores are each
         entry's own sigmoid instead of a softmax over the entries. renorm False: the chosen scores are the weights as they are.
         table_vocab > 0: there is no router; row `token id` of `table` [table_vocab, top] (integers) names the token's experts,
         each with the weight 1 / top, and forward() takes the token ids. shared_gate False: the shared expert is added as it is.
-        corrected False: choices go by the scores themselves (no `correction` tensor)."""
+        corrected False: choices go by the scores themselves (no `correction` tensor). router_bias: the logits are W_r h + `router.b`."""
         super().__init__()
         self.table_vocab, self.shared_gate = int(table_vocab), bool(shared_gate) and not table_vocab
         self.gated, self.sigmoid, self.renorm = bool(gated), bool(sigmoid), bool(renorm)
@@ -758,6 +819,7 @@ class RoutedExperts(nn.Module):
         else:
             self.router = _param(total + (1 if shared_ff and self.shared_gate else 0), width, dtype=torch.float32)
             self.correction = _param(total, dtype=torch.float32) if corrected else None
+            self.router_b = _param(self.router.shape[0], dtype=torch.float32) if router_bias else None      # (0 for the shared gate's row)
         self.w_gu, self.w_down = _param(experts, (2 if gated else 1) * ff, width), _param(experts, width, ff)
         if shared_ff:
             self.s_gu, self.s_down = _param(2 * shared_ff, width), _param(width, shared_ff)
@@ -768,6 +830,8 @@ class RoutedExperts(nn.Module):
             {"router": _copy_into(self.router[:total])}
         if not self.table_vocab and self.correction is not None:
             out["correction"] = _copy_into(self.correction)
+        if not self.table_vocab and self.router_b is not None:
+            out["router.b"] = _copy_into(self.router_b[:total])
         for e in range(self.E):
             if self.gated:
                 out[f"e{e}.gate"] = _copy_into(self.w_gu[e, :ff])
@@ -783,15 +847,16 @@ class RoutedExperts(nn.Module):
                 out["shared.sg"] = _copy_into(self.router[total:])
         return out
 
-    def forward(self, xh: torch.Tensor, tokens: torch.Tensor | None = None, res: torch.Tensor | None = None) -> torch.Tensor:
-        """The mixture's output; with `res` (the 32-bit residual) it is added there and the new residual is returned instead."""
+    def parts(self, xh: torch.Tensor, tokens: torch.Tensor | None = None, wide: torch.Tensor | None = None) -> tuple:
+        """What a token's output is summed from: (expert rows, plan, weights, the shared expert's output or None, the pre-activation of its
+        gate or None). wide: the layer's input in 32-bit, for the router (default: xh)."""
         n, width = xh.shape
         total = self.E + self.ident
         if self.table_vocab:
             z = None
             ids, wts = ops_seq.moe_table_route(tokens, self.table, 1.0 / self.top)
         else:
-            z = F.linear(xh.float(), self.router)                                 # 32-bit, [n, total (+ 1: the shared gate)]
+            z = F.linear(wide if wide is not None else xh.float(), self.router, self.router_b)      # 32-bit, [n, total (+ 1: the shared gate)]
             ids, wts = ops_seq.moe_route(z, total, self.correction, self.top, self.count, self.keep, self.scale, self.sigmoid, self.renorm)
         per_expert = n * self.top // self.E                 # rows an expert gets on average: the tile height follows it
         plan = ops_seq.moe_plan(ids, self.E, 128 if per_expert >= 256 else (64 if per_expert >= 64 else 16))
@@ -804,10 +869,15 @@ class RoutedExperts(nn.Module):
             sact = torch.empty(n, self.shared_ff, dtype=xh.dtype, device=xh.device)
             ops_seq.glu_act(F.linear(xh, self.s_gu), self.shared_ff, sact, kind=0)
             shared, gate = F.linear(sact, self.s_down), (z[:, total:] if self.shared_gate else None)
+        return rows, plan, wts, shared, gate
+
+    def forward(self, xh: torch.Tensor, tokens: torch.Tensor | None = None, res: torch.Tensor | None = None) -> torch.Tensor:
+        """The mixture's output; with `res` (the 32-bit residual) it is added there and the new residual is returned instead."""
+        rows, plan, wts, shared, gate = self.parts(xh, tokens)
         if res is not None and xh.dtype == torch.float32:
             ops_seq.moe_combine(rows, plan, wts, xh, shared, gate, None, res)
             return res
-        out = torch.empty(n, width, dtype=xh.dtype, device=xh.device)
+        out = torch.empty(xh.shape, dtype=xh.dtype, device=xh.device)
         ops_seq.moe_combine(rows, plan, wts, xh, shared, gate, out, res)
         return out
 

@@ -15,7 +15,7 @@ import torch
 
 from . import build as _build
 
-ABI_VERSION = 6
+ABI_VERSION = 7
 _P, _I, _L, _F = c_void_p, c_int, c_int64, c_float
 
 SIGNATURES = {
@@ -43,6 +43,8 @@ SIGNATURES = {
     "nvs_shift_norm": (c_int, [_P, _P, _P, _P, _P, _I, _P, _P, _P, _P, _I, _L, _I, _F, _P, _P, _P, _P]),
     "nvs_gated_lookup": (c_int, [_P, _L, _P, _L, _L, _I, _P, _I, _L, _P, _P]),
     "nvs_qk_rows": (c_int, [_P, _L, _I, _P, _P, _L, _I, _P, _F, _I, _I, _I, _I, _P, _P, _P, _I, _L, _P, _P, _P, _I, _I, _P, _L, _P, _P, _P, _P]),
+    "nvs_branch_norm": (c_int, [_P, _P, _P, _L, _P, _P, _I, _I, _L, _P, _P, _I, _F, _P, _P]),
+    "nvs_qkv_store": (c_int, [_P, _P, _P, _L, _I, _I, _I, _I, _I, _P, _P, _I, _I, _F, _I, _F, _F, _P, _L, _P, _I, _P, _L, _P, _P, _P]),
     "nvs_pool_rows": (c_int64, [_I, _I]),
     "nvs_pool_blocks": (c_int, [_P, _P, _I, _I, _I, _I, _I, _I, _P, _P, _P, _L, _P, _L, _P, _P, _P]),
     "nvs_knorm_kvstore": (c_int, [_P, _P, _L, _I, _P, _F, _I, _I, _I, _I, _P, _P, _P, _I, _L, _P, _P, _P]),
@@ -260,6 +262,26 @@ def knorm_kvstore(k: torch.Tensor, v: torch.Tensor, knorm: torch.Tensor | None, 
                                  _rotation(rot_freq), n, _ptr(k_cache), _ptr(v_cache), _stream()))
 
 
+def qkv_store(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, H: int, G: int, d: int, dv: int, block_size: int, slots: torch.Tensor, k_cache,
+              v_cache, pos: torch.Tensor | None, rot: "Rotation | None", unit: bool, eps: float, q_scale: float,
+              first: torch.Tensor | None = None, mix: torch.Tensor | None = None):
+    """q [n, H*d], k [n, G*d], v [n, G*dv]: column ranges of ONE projection output. Queries and keys are rotated, then (unit) divided by their
+    root mean square per head; queries, times q_scale, are rewritten in place, keys and values stored. first [n, G*dv] and mix (one 32-bit
+    number): the values stored are (1 - mix) v + mix first."""
+    lib = load_library()
+    n = q.shape[0]
+    assert q.shape == (n, H * d) and k.shape == (n, G * d) and v.shape == (n, G * dv) and q.stride(1) == k.stride(1) == v.stride(1) == 1
+    assert q.stride(0) == k.stride(0) == v.stride(0) and slots.dtype == torch.int32 and slots.numel() >= n
+    assert k_cache.is_contiguous() and v_cache.is_contiguous() and k_cache.shape[0] % block_size == 0
+    assert tuple(k_cache.shape[1:]) == (G, d) and tuple(v_cache.shape[1:]) == (G, dv)
+    assert rot is None or (pos is not None and pos.dtype == torch.int64 and pos.numel() >= n and pos.is_contiguous() and rot.dims <= d)
+    assert first is None or (first.shape == v.shape and first.stride(1) == 1 and mix.dtype == torch.float32 and mix.numel() == 1)
+    _check(lib.nvs_qkv_store(_ptr(q), _ptr(k), _ptr(v), q.stride(0), _same(q, k, v, first, k_cache, v_cache), H, G, d, dv,
+                             _ptr(pos) if rot else None, _ptr(rot.freq) if rot else None, rot.dims if rot else 0, int(rot.halves) if rot else 0,
+                             rot.mag if rot else 1.0, int(unit), eps, q_scale, _ptr(first), first.stride(0) if first is not None else 0,
+                             _ptr(mix) if first is not None else None, block_size, _ptr(slots), n, _ptr(k_cache), _ptr(v_cache), _stream()))
+
+
 def window_attn(q: torch.Tensor, qnorm: torch.Tensor | None, eps: float, gate: torch.Tensor | None, k_cache, v_cache,
                 block_tables: torch.Tensor, block_size: int, por: Portions, H: int, G: int, d: int, dv: int, scale: float,
                 window: int, out: torch.Tensor, chunk: int = 0, rot_freq: torch.Tensor | None = None, gate_per_head: bool = False,
@@ -436,6 +458,25 @@ def offset_norm_rows(x: torch.Tensor, rows: torch.Tensor | None, nrows: int, w: 
     assert rows is not None or nrows <= x.shape[0]
     _check(lib.nvs_sandwich_norm(_ptr(x), _ptr(a), 1.0, None, 1.0, _ptr(wa), _ptr(rows), nrows, _ptr(w), w_off, _same(out, w, a, wa), x.shape[1],
                                  eps, _ptr(sums), _ptr(out), _stream()))
+
+
+def branch_norm(x: torch.Tensor, a: torch.Tensor | None, w: torch.Tensor, ls: torch.Tensor | None, eps: float, out: torch.Tensor | None,
+                chosen: "tuple | None" = None):
+    """x += rms(y) * w * ls (in place; ls None: no scale), y = a (may be None) + with chosen = (rows, plan, weights) of a routed layer the
+    weighted sum of every token's choices; out (may be None) receives the new x in the activation type."""
+    lib = load_library()
+    n, width = x.shape
+    rows, plan, wts = chosen if chosen is not None else (None, None, None)
+    assert x.dtype == torch.float32 and x.is_contiguous() and w.numel() == width and (ls is None or ls.numel() == width)
+    assert a is None or (a.shape == x.shape and a.is_contiguous())
+    assert out is None or (out.shape == x.shape and out.is_contiguous())
+    top = 0
+    if rows is not None:
+        top = wts.shape[1]
+        assert rows.stride(1) == 1 and rows.shape[1] == width and wts.dtype == torch.float32 and wts.is_contiguous()
+        assert wts.shape[0] == n and plan.pair_row.shape == (n, top)
+    _check(lib.nvs_branch_norm(_ptr(x), _ptr(a), _ptr(rows), rows.stride(0) if rows is not None else 0, _ptr(plan.pair_row) if plan else None,
+                               _ptr(wts), top, _same(w, a, rows, ls, out), n, _ptr(w), _ptr(ls), width, eps, _ptr(out), _stream()))
 
 
 def gated_memory_scan(proj: torch.Tensor, v_col: int, k_col: int, q_col: int, i_col: int, f_col: int, i_bias: torch.Tensor,

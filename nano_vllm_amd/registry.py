@@ -89,6 +89,17 @@ def _ligidra_build(config, dtype=None):
     return LigidraForCausalLM(config, dtype)
 
 
+def _reselorn_config(path: str, raw: dict):
+    from .reselorn import ReselornConfig
+    from .weights import checkpoint_shapes
+    return ReselornConfig(raw, checkpoint_shapes(path))
+
+
+def _reselorn_build(config, dtype=None):
+    from .reselorn import ReselornForCausalLM
+    return ReselornForCausalLM(config, dtype)
+
+
 REGISTRY: dict[str, ModelSpec] = {
     "Qwen3ForCausalLM": ModelSpec("Qwen3ForCausalLM", _qwen3_config, _qwen3_build),
     "Qwen2ForCausalLM": ModelSpec("Qwen2ForCausalLM", _qwen3_config, _qwen3_build),      # same module tree, biased qkv, no q/k norm
@@ -102,6 +113,8 @@ REGISTRY: dict[str, ModelSpec] = {
                          dtypes=("bfloat16", "float32")),
     "Ligidra": ModelSpec("Ligidra", _ligidra_config, _ligidra_build, stateful=True, block_multiple=16,
                          dtypes=("bfloat16", "float32")),
+    "Reselorn": ModelSpec("Reselorn", _reselorn_config, _reselorn_build, stateful=True, block_multiple=16,
+                          dtypes=("bfloat16", "float32")),
 }
 
 
