@@ -43,6 +43,22 @@ __global__ void embed_sinusoid_kernel(const T* __restrict__ table, const int64_t
   }
 }
 
+// without a sinusoid: table rows times scale, four columns per access
+template <typename T>
+__global__ void embed_rows_kernel(const T* __restrict__ table, const int64_t* __restrict__ ids, int width, float scale, float* __restrict__ x,
+                                  T* __restrict__ xh) {
+  const int64_t t = blockIdx.x;
+  const T* row = table + ids[t] * width;
+  for (int c = threadIdx.x * 4; c < width; c += blockDim.x * 4) {
+    float v[4];
+    ldv<4>(row + c, v);
+#pragma unroll
+    for (int e = 0; e < 4; ++e) v[e] *= scale;
+    stv<4>(x + t * width + c, v);
+    if (xh) stv<4>(xh + t * width + c, v);
+  }
+}
+
 // one workgroup per token row
 template <typename T>
 __global__ void norm_residual_kernel(const T* __restrict__ m, const T* __restrict__ m2, const T* __restrict__ w1,
@@ -571,6 +587,11 @@ extern "C" int nvs_embed_sinusoid(const void* table, int dtype, const int64_t* i
                                   float scale, float base, float* x, void* xh, void* stream) {
   NVS_REQUIRE(table && ids && pos && x && n >= 0 && width > 0 && (base > 1.f || base == 0.f), "nvs_embed_sinusoid: bad argument");
   if (n == 0) return NVS_OK;
+  if (base == 0.f && width % 4 == 0 && ((uintptr_t)table | (uintptr_t)x | (uintptr_t)xh) % 16 == 0) {
+    NVS_DISPATCH(dtype, embed_rows_kernel<T><<<dim3((unsigned)n), dim3(width >= 1024 ? 256 : ((width + 255) / 256) * 64), 0, (hipStream_t)stream>>>(
+                            (const T*)table, ids, width, scale, x, (T*)xh));
+    return nvs_check_launch("nvs_embed_sinusoid (rows)");
+  }
   NVS_DISPATCH(dtype, embed_sinusoid_kernel<T><<<dim3((unsigned)n), dim3(threads_for(width)), 0, (hipStream_t)stream>>>(
                           (const T*)table, ids, pos, width, scale, base > 1.f ? log2f(base) : 0.f, x, (T*)xh));
   return nvs_check_launch("nvs_embed_sinusoid");

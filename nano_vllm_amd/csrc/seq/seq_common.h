@@ -70,7 +70,7 @@ __device__ __forceinline__ void stv(bf16_t* p, const float (&v)[VEC]) {
   }
 }
 
-// N (1, 2 or 4) consecutive elements in one piece (the address is aligned to the piece)
+// N (a power of two up to 8) consecutive elements in one piece (the address is aligned to the piece)
 template <int N, typename T>
 __device__ __forceinline__ void ldp(const T* p, float (&v)[N]) {
   typedef __attribute__((ext_vector_type(N))) T vec_t;

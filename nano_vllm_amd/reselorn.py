@@ -46,7 +46,7 @@ class ReselornConfig:
         self.eps = float(raw["norm"]["eps"])
         self.max_position_embeddings = 1 << 24          # positions are exact integers in a 32-bit float up to here
         self.eos_token_id = raw.get("eos_token_id", -1)
-        first = None                                    # (layer, value columns) of the first value-mixing layer
+        first = None                                    # (layer, its value heads) of the first value-mixing layer
         for i, layer in enumerate(self.layers):
             if layer["type"] != "attention":
                 raise ValueError(f"layer {i}: unknown mixer type {layer['type']!r}")
@@ -57,9 +57,9 @@ class ReselornConfig:
             if heads % kv_heads:
                 raise ValueError(f"layer {i}: {heads} query heads do not share {kv_heads} key/value heads evenly")
             if layer["mixer"].get("v_mix"):
-                first = first or (i, kv_heads * vdim)
-                if first[1] != kv_heads * vdim:
-                    raise ValueError(f"layer {i}: its values have {kv_heads * vdim} columns, those of layer {first[0]}, which they are mixed with, {first[1]}")
+                first = first or (i, (kv_heads, vdim))
+                if first[1] != (kv_heads, vdim):
+                    raise ValueError(f"layer {i}: values of {kv_heads} x {vdim} cannot be mixed with those of layer {first[0]}, {first[1][0]} x {first[1][1]}")
 
 
 def head_sizes(m: dict) -> tuple[int, int, int, int]:

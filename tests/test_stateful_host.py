@@ -492,3 +492,72 @@ def test_every_block_of_positions_has_a_place_of_its_own_in_the_pages(block, poo
         seen.add((page, at))
         for b in range(8 * u, 8 * u + 8):
             assert page <= (b * pool + pool - 1) // block
+
+
+# ---- Reselorn -------------------------------------------------------------------------------------------------------------
+def rsl_raw():
+    moe = {"kind": "moe", "expert": {"ff": 10}, "router": {"experts": 3, "top": 2}, "shared": {"ff": 12}}
+    att = {"heads": 4, "kv_heads": 2, "dim": 6, "vdim": 5, "scale": 0.4, "mask": {"size": 10}, "v_mix": True,
+           "rot": {"dims": 4, "base": 100.0, "scaling": {"factor": 2.0, "fast": 2.0, "slow": 0.5, "original": 16}}}
+    return {"architecture": "Reselorn", "norm": {"eps": 1e-5}, "vocab": 29, "width": 16,
+            "layers": [{"type": "attention", "mixer": dict(att, v_mix=False, heads=3, kv_heads=3, rot=None, mask=None), "mlp": {"kind": "dense", "ff": 9}},
+                       {"type": "attention", "mixer": att, "mlp": moe}, {"type": "attention", "mixer": dict(att, dim=8), "mlp": None},
+                       {"type": "attention", "mixer": dict(att, heads=2), "mlp": dict(moe, shared=None)}]}
+
+
+def test_reselorn_registry_and_config_checks(tmp_path):
+    from nano_vllm_amd.registry import REGISTRY, resolve
+    (tmp_path / "config.json").write_text(json.dumps(rsl_raw()))
+    spec, cfg = resolve(str(tmp_path))
+    assert spec is REGISTRY["Reselorn"] and spec.stateful and set(spec.dtypes) == {"bfloat16", "float32"}
+    assert (cfg.vocab_size, cfg.hidden_size, cfg.num_hidden_layers, cfg.eps) == (29, 16, 4, 1e-5)
+    cases = [(lambda r: r["layers"][0].update(type="lstm"), "mixer type"), (lambda r: r["layers"][0].update(mlp={"kind": "table"}), "feed-forward kind"),
+             (lambda r: r["layers"][1]["mixer"].update(kv_heads=3), "evenly"), (lambda r: r["layers"][3]["mixer"].update(vdim=7), "mixed with"),
+             (lambda r: r["layers"][3]["mixer"].update(kv_heads=1, vdim=10), "mixed with")]
+    for change, msg in cases:
+        raw = json.loads(json.dumps(rsl_raw()))
+        change(raw)
+        (tmp_path / "config.json").write_text(json.dumps(raw))
+        with pytest.raises(ValueError, match=msg):
+            resolve(str(tmp_path))
+    raw = rsl_raw()
+    raw["layers"][0]["mixer"]["vdim"] = 13                      # (a layer that does not mix may have other sizes)
+    (tmp_path / "config.json").write_text(json.dumps(raw))
+    resolve(str(tmp_path))
+
+
+def test_reselorn_checkpoint_names_loaders_and_layout(tmp_path):
+    import math
+
+    from nano_vllm_amd.registry import resolve
+    from nano_vllm_amd.reselorn import ReselornConfig, ReselornForCausalLM, random_tensors, tensor_shapes, write_synthetic_checkpoint
+    from nano_vllm_amd.weights import load_model
+    raw = rsl_raw()
+    model = ReselornForCausalLM(ReselornConfig(raw), torch.float32, block_size=16)
+    loaders, shapes = model.named_loaders(), tensor_shapes(raw)
+    assert set(loaders) == set(shapes) and "head" not in shapes
+    assert not any(n in shapes for n in ("l0.mix.vmix", "l2.norm2", "l2.ls2", "l3.mlp.shared.up", "l1.mlp.correction", "l1.mlp.shared.sg", "l1.mix.q.norm"))
+    tensors = random_tensors(raw, seed=3)
+    with torch.no_grad():
+        for name, t in tensors.items():
+            assert tuple(t.shape) == tuple(shapes[name])
+            loaders[name](t)
+    assert sum(p.numel() for p in model.parameters()) == sum(math.prod(s) for s in shapes.values())
+    f = lambda n: tensors[n].float()
+    a, b = model.layers[1].mixer, model.layers[0].mixer
+    assert a.in_w.shape == (24 + 12 + 10, 16) and a.in_b is None and torch.equal(a.in_w[24:36], f("l1.mix.k")) and torch.equal(a.in_w[36:], f("l1.mix.v"))
+    assert torch.equal(a.attn.sink, f("l1.mix.sink")) and float(a.attn.vmix) == float(f("l1.mix.vmix")) and a.attn.vmix.dtype == torch.float32
+    assert b.attn.vmix is None and b.attn.rot_freq is None and b.attn.window == 0 and a.attn.window == 10 and a.attn.q_norm is None
+    assert a.attn.kv_shapes() == ((2, 6), (2, 5)) and a.attn.page_shapes() == {} and a.attn.rot_mag == pytest.approx(1 + 0.1 * math.log(2.0))
+    moe = model.layers[1].mlp
+    assert torch.equal(moe.router_b, f("l1.mlp.router.b")) and torch.equal(moe.router, f("l1.mlp.router")) and moe.correction is None
+    assert torch.equal(moe.w_gu[2, 10:], f("l1.mlp.e2.up")) and torch.equal(model.layers[0].mlp.gu[:9], f("l0.mlp.gate"))
+    assert torch.equal(model.layers[1].norm2.scale, f("l1.ls2")) and torch.equal(model.layers[3].norm1.w, f("l3.norm1")) and model.layers[2].norm2 is None
+    # a checkpoint may hold tensors of what a layer leaves out; any other unknown tensor is an error, and so is a missing one
+    extra = dict(tensors, **{"l2.norm2": torch.ones(16), "l2.ls2": torch.ones(16), "l0.mix.vmix": torch.tensor(0.5)})
+    path = write_synthetic_checkpoint(str(tmp_path / "a"), raw, tensors=extra)
+    assert load_model(ReselornForCausalLM(resolve(path)[1], torch.float32, block_size=16), path) == len(extra)
+    for bad in (dict(tensors, **{"l2.mlp.up": torch.ones(2)}), {k: v for k, v in tensors.items() if k != "l3.ls1"}):
+        path = write_synthetic_checkpoint(str(tmp_path / "b"), raw, tensors=bad)
+        with pytest.raises(KeyError):
+            load_model(ReselornForCausalLM(resolve(path)[1], torch.float32, block_size=16), path)
